@@ -49,61 +49,127 @@ __device__ __forceinline__ int first_visible(int pos, const WindowTerms& t) {
 // cos_t, sin_t [positions][rot / 2] (or null): after the norm the first `rot` values of a q or k head are turned, value
 // i < rot / 2 paired with value i + rot / 2 (with `pairs`: value 2 i with value 2 i + 1), by the angle whose cosine
 // and sine stand at [position][i].  Without write_kv the rows hold queries only (keys and values are another layer's).
+// v_col: the column where the rows' values start: behind the keys, or, for a layer whose values are its keys as projected
+// (before norm and rotation; vdim == dim, nv == nkv), where the keys start.
+// temp_coef != 0: queries at position p are multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1), after norm and
+// rotation.
+struct IntakeArgs {
+  const float* proj;
+  int width;
+  const float* bias;
+  const int* page_table;
+  int table_stride;
+  const int* tok_seq;
+  const int* tok_pos;
+  const float* q_gain;
+  const float* k_gain;
+  float eps;
+  const float* cos_t;
+  const float* sin_t;
+  int rot, pairs, nh, nkv, nv, dim, vdim, write_kv, v_col;
+  float temp_coef;
+  int temp_every;
+};
+
+// where an item's values stand in the projection's rows; its kind
+struct IntakeItem {
+  bool is_q, is_k;
+  int len, col;
+};
+__device__ __forceinline__ IntakeItem intake_item(const IntakeArgs& a, int item) {
+  IntakeItem t;
+  t.is_q = item < a.nh, t.is_k = !t.is_q && item < a.nh + a.nkv;
+  t.len = (t.is_q || t.is_k) ? a.dim : a.vdim;
+  t.col = t.is_q ? item * a.dim : (t.is_k ? a.nh * a.dim + (item - a.nh) * a.dim : a.v_col + (item - a.nh - a.nkv) * a.vdim);
+  return t;
+}
+
+// One wave stores one item of a token: scaled by inv with its gain (null: neither), turned, with a query's temperature.
 template <typename T>
-__global__ void window_intake_kernel(const float* __restrict__ proj, int width, const float* __restrict__ bias,
-                                     T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages,
-                                     const int* __restrict__ page_table, int table_stride,
-                                     const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
-                                     const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
-                                     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, int pairs,
-                                     int nh, int nkv, int nv, int dim, int vdim, int write_kv) {
-  const int wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE;
-  const int tok = blockIdx.x;
-  const int item = blockIdx.y * (blockDim.x / SYN_WAVE) + wave;
-  if (item >= (write_kv ? nh + nkv + nv : nh)) return;
-  const bool is_q = item < nh, is_k = !is_q && item < nh + nkv;
-  const int len = (is_q || is_k) ? dim : vdim;
-  const int col = is_q ? item * dim : (is_k ? nh * dim + (item - nh) * dim : (nh + nkv) * dim + (item - nh - nkv) * vdim);
-  const float* src = proj + (size_t)tok * width + col;
-  const float* b = bias ? bias + col : nullptr;
-  const float* gain = is_q ? q_gain : (is_k ? k_gain : nullptr);
-  float inv = 1.f;
-  if (gain) {
-    float ss = 0.f;
-    for (int d = lane; d < len; d += SYN_WAVE) {
-      const float v = src[d] + (b ? b[d] : 0.f);
-      ss += v * v;
-    }
-    inv = 1.f / sqrtf(wave_sum(ss) / (float)len + eps);
-  }
-  const int pos = tok_pos[tok];
+__device__ __forceinline__ void intake_store(const IntakeArgs& a, const IntakeItem& t, int tok, int item, int lane,
+                                             const float* gain, float inv, T* __restrict__ q_out, T* __restrict__ k_pages,
+                                             T* __restrict__ v_pages) {
+  const float* src = a.proj + (size_t)tok * a.width + t.col;
+  const float* b = a.bias ? a.bias + t.col : nullptr;
+  const int pos = a.tok_pos[tok];
   T* dst;
   size_t stride = 1;
-  if (is_q) {
-    dst = q_out + ((size_t)tok * nh + item) * dim;
+  float temp = 1.f;
+  if (t.is_q) {
+    dst = q_out + ((size_t)tok * a.nh + item) * a.dim;
+    if (a.temp_coef != 0.f) temp = 1.f + a.temp_coef * logf((float)((pos + 1) / a.temp_every + 1));
   } else {
-    const int page = page_table[(size_t)tok_seq[tok] * table_stride + pos / SYN_PAGE];
-    if (is_k) {
-      dst = k_pages + (((size_t)page * nkv + (item - nh)) * SYN_PAGE + pos % SYN_PAGE) * dim;
+    const int page = a.page_table[(size_t)a.tok_seq[tok] * a.table_stride + pos / SYN_PAGE];
+    if (t.is_k) {
+      dst = k_pages + (((size_t)page * a.nkv + (item - a.nh)) * SYN_PAGE + pos % SYN_PAGE) * a.dim;
     } else {
-      dst = v_pages + ((size_t)page * nv + (item - nh - nkv)) * vdim * SYN_PAGE + pos % SYN_PAGE;
+      dst = v_pages + ((size_t)page * a.nv + (item - a.nh - a.nkv)) * a.vdim * SYN_PAGE + pos % SYN_PAGE;
       stride = SYN_PAGE;
     }
   }
-  const int half = (cos_t && (is_q || is_k)) ? rot / 2 : 0;
-  for (int d = lane; d < len; d += SYN_WAVE) {
+  const int half = (a.cos_t && (t.is_q || t.is_k)) ? a.rot / 2 : 0;
+  for (int d = lane; d < t.len; d += SYN_WAVE) {
     float v = src[d] + (b ? b[d] : 0.f);
     if (gain) v = v * inv * gain[d];
     if (d < 2 * half) {
-      const bool first = pairs ? d % 2 == 0 : d < half;
-      const int i = pairs ? d / 2 : (first ? d : d - half);
-      const int mate = pairs ? (d ^ 1) : (first ? d + half : d - half);
+      const bool first = a.pairs ? d % 2 == 0 : d < half;
+      const int i = a.pairs ? d / 2 : (first ? d : d - half);
+      const int mate = a.pairs ? (d ^ 1) : (first ? d + half : d - half);
       float o = src[mate] + (b ? b[mate] : 0.f);
       if (gain) o = o * inv * gain[mate];
-      const float c = cos_t[(size_t)pos * half + i], sn = sin_t[(size_t)pos * half + i];
+      const float c = a.cos_t[(size_t)pos * half + i], sn = a.sin_t[(size_t)pos * half + i];
       v = first ? v * c - o * sn : v * c + o * sn;
     }
-    dst[(size_t)d * stride] = from_f32<T>(v);
+    dst[(size_t)d * stride] = from_f32<T>(v * temp);
+  }
+}
+
+// norms (if any) over each head, one gain [dim] for all heads
+template <typename T>
+__global__ void window_intake_kernel(IntakeArgs a, T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages) {
+  const int wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE;
+  const int tok = blockIdx.x;
+  const int item = blockIdx.y * (blockDim.x / SYN_WAVE) + wave;
+  if (item >= (a.write_kv ? a.nh + a.nkv + a.nv : a.nh)) return;
+  const IntakeItem t = intake_item(a, item);
+  const float* gain = t.is_q ? a.q_gain : (t.is_k ? a.k_gain : nullptr);
+  float inv = 1.f;
+  if (gain) {
+    const float* src = a.proj + (size_t)tok * a.width + t.col;
+    const float* b = a.bias ? a.bias + t.col : nullptr;
+    float ss = 0.f;
+    for (int d = lane; d < t.len; d += SYN_WAVE) {
+      const float v = src[d] + (b ? b[d] : 0.f);
+      ss += v * v;
+    }
+    inv = 1.f / sqrtf(wave_sum(ss) / (float)t.len + a.eps);
+  }
+  intake_store<T>(a, t, tok, item, lane, gain, inv, q_out, k_pages, v_pages);
+}
+
+// norms over all query heads at once and over all key heads at once (gains [nh * dim] and [nkv * dim]): a workgroup a
+// token, which sums both squares first and then stores item after item
+template <typename T>
+__global__ void __launch_bounds__(512)
+window_intake_whole_kernel(IntakeArgs a, T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages) {
+  __shared__ float red[16];
+  const int wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE, n_waves = blockDim.x / SYN_WAVE;
+  const int tok = blockIdx.x, nq = a.nh * a.dim, nk = a.write_kv ? a.nkv * a.dim : 0;
+  const float* row = a.proj + (size_t)tok * a.width;
+  float sq = 0.f, sk = 0.f;
+  for (int d = threadIdx.x; d < nq + nk; d += blockDim.x) {
+    const float v = row[d] + (a.bias ? a.bias[d] : 0.f);
+    if (d < nq) sq = fmaf(v, v, sq);
+    else sk = fmaf(v, v, sk);
+  }
+  sq = block_sum(sq, red);
+  if (nk) sk = block_sum(sk, red);       // (the same for the whole workgroup)
+  const float inv_q = 1.f / sqrtf(sq / (float)nq + a.eps), inv_k = nk ? 1.f / sqrtf(sk / (float)nk + a.eps) : 1.f;
+  const int items = a.write_kv ? a.nh + a.nkv + a.nv : a.nh;
+  for (int item = wave; item < items; item += n_waves) {
+    const IntakeItem t = intake_item(a, item);
+    const float* gain = t.is_q ? a.q_gain + item * a.dim : (t.is_k ? a.k_gain + (item - a.nh) * a.dim : nullptr);
+    intake_store<T>(a, t, tok, item, lane, gain, t.is_q ? inv_q : inv_k, q_out, k_pages, v_pages);
   }
 }
 
@@ -111,25 +177,32 @@ SYN_EXPORT int syn_window_intake(const float* proj, int width, const float* bias
                                  void* v_pages, int is_f32, const int* page_table, int table_stride, const int* tok_seq,
                                  const int* tok_pos, const float* q_gain, const float* k_gain, float eps,
                                  const float* cos_t, const float* sin_t, int rot, int pairs, int n_tokens,
-                                 int nh, int nkv, int nv, int dim, int vdim, int write_kv, hipStream_t stream) {
+                                 int nh, int nkv, int nv, int dim, int vdim, int write_kv, int norm_whole,
+                                 int values_are_keys, float temp_coef, int temp_every, hipStream_t stream) {
   SYN_CHECK(n_tokens > 0 && nh > 0 && nkv > 0 && nv > 0 && dim > 0 && vdim > 0, "window_intake: empty input");
-  SYN_CHECK(width >= (write_kv ? (nh + nkv) * dim + nv * vdim : nh * dim), "window_intake: rows of %d values do not hold q%s",
-            width, write_kv ? ", k and v" : "");
+  SYN_CHECK(!values_are_keys || (nv == nkv && vdim == dim), "window_intake: values that are the keys have their heads and sizes");
+  SYN_CHECK(width >= (write_kv ? (nh + nkv) * dim + (values_are_keys ? 0 : nv * vdim) : nh * dim),
+            "window_intake: rows of %d values do not hold q%s", width, write_kv ? ", k and v" : "");
   SYN_CHECK((q_gain == nullptr) == (k_gain == nullptr), "window_intake: q and k gains come together");
+  SYN_CHECK(!norm_whole || q_gain, "window_intake: a norm over all heads without its gains");
+  SYN_CHECK(temp_coef == 0.f || temp_every > 0, "window_intake: a temperature that steps every %d positions", temp_every);
   SYN_CHECK((cos_t == nullptr) == (sin_t == nullptr) && (cos_t == nullptr || (rot > 0 && rot % 2 == 0 && rot <= dim)),
             "window_intake: a rotation of %d of %d values", rot, dim);
   const int wpb = 4, items = write_kv ? nh + nkv + nv : nh;
+  const IntakeArgs a = {proj, width, bias, page_table, table_stride, tok_seq, tok_pos, q_gain, k_gain, eps, cos_t, sin_t,
+                        rot, pairs, nh, nkv, nv, dim, vdim, write_kv, values_are_keys ? nh * dim : (nh + nkv) * dim,
+                        temp_coef, temp_every};
+  if (norm_whole) {
+    if (is_f32) window_intake_whole_kernel<float><<<n_tokens, 512, 0, stream>>>(a, (float*)q_out, (float*)k_pages, (float*)v_pages);
+    else window_intake_whole_kernel<bf16><<<n_tokens, 512, 0, stream>>>(a, (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages);
+    SYN_LAUNCH_CHECK("window_intake_whole");
+    return 0;
+  }
   const dim3 grid(n_tokens, (items + wpb - 1) / wpb);
   if (is_f32)
-    window_intake_kernel<float><<<grid, wpb * SYN_WAVE, 0, stream>>>(proj, width, bias, (float*)q_out, (float*)k_pages,
-                                                                     (float*)v_pages, page_table, table_stride, tok_seq,
-                                                                     tok_pos, q_gain, k_gain, eps, cos_t, sin_t, rot, pairs,
-                                                                     nh, nkv, nv, dim, vdim, write_kv);
+    window_intake_kernel<float><<<grid, wpb * SYN_WAVE, 0, stream>>>(a, (float*)q_out, (float*)k_pages, (float*)v_pages);
   else
-    window_intake_kernel<bf16><<<grid, wpb * SYN_WAVE, 0, stream>>>(proj, width, bias, (bf16*)q_out, (bf16*)k_pages,
-                                                                    (bf16*)v_pages, page_table, table_stride, tok_seq,
-                                                                    tok_pos, q_gain, k_gain, eps, cos_t, sin_t, rot, pairs,
-                                                                    nh, nkv, nv, dim, vdim, write_kv);
+    window_intake_kernel<bf16><<<grid, wpb * SYN_WAVE, 0, stream>>>(a, (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages);
   SYN_LAUNCH_CHECK("window_intake");
   return 0;
 }
@@ -408,6 +481,7 @@ window_prefill_bf16_kernel(const bf16* __restrict__ q, const bf16* __restrict__ 
   const float r1 = terms.r1 ? terms.r1[head] : 0.f, r2 = terms.r1 ? terms.r2[head] : 0.f;
   constexpr float LOG2E = 1.4426950408889634f;
   const float scale2 = scale * LOG2E, slope2 = slope * LOG2E, cap2 = terms.softcap * LOG2E;
+  const float cap_in = terms.softcap > 0.f ? 2.f / terms.softcap : 0.f;     // (a score in units of ln 2 -> 2 z log2 e)
   // (the sink's score in units of ln 2; a score of 0 is 0 in any unit)
   float m = terms.sinks ? terms.sinks[head] * LOG2E : (terms.sink_one ? 0.f : -INFINITY);
   float l = (terms.sinks || terms.sink_one) ? 1.f : 0.f;
@@ -485,7 +559,8 @@ window_prefill_bf16_kernel(const bf16* __restrict__ q, const bf16* __restrict__ 
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         float v = s[t][e] * scale2;
-        if (terms.softcap > 0.f) v = cap2 * tanhf(s[t][e] * scale / terms.softcap);
+        if (terms.softcap > 0.f)      // cap tanh(z) = cap (1 - 2 / (exp(2 z) + 1)), good to cap * 2^-23
+          v = fmaf(-2.f * cap2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * cap_in) + 1.f), cap2);
         const float dist = dist0 - (float)(16 * t + e);          // query position - key position
         if (slope2 != 0.f) v -= slope2 * dist;
         if (terms.r1) v -= r1 * __builtin_amdgcn_logf(fmaf(r2, dist, 1.f));

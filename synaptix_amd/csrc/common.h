@@ -130,6 +130,18 @@ __device__ __forceinline__ float gated(int act, float gate, float up, float limi
   return gate_activation(act, gate) * up;
 }
 
+// ---- the activation of an ungated feed-forward, on the 32-bit sums of its first product ----
+#define SYN_POINT_NONE 0
+#define SYN_POINT_RELU_SQUARED 1
+#define SYN_POINT_COUNT 2
+__device__ __forceinline__ float point_activation(int point, float z) {
+  if (point == SYN_POINT_RELU_SQUARED) {
+    z = z > 0.f ? z : (z <= 0.f ? 0.f : z);      // (a NaN stays one)
+    z *= z;
+  }
+  return z;
+}
+
 // ---- what an attention kernel may do to a scaled score before the mask and the softmax ----
 // A soft cap, cap * tanh(score / cap), and a penalty in the distance between query and key, - slope[head] * (q - k)
 // (the linear bias of crates/synaptix-ops/src/pos/alibi.rs:47-66 for keys at or before the query).  Neither is set

@@ -196,15 +196,15 @@ SYN_EXPORT int syn_add_rmsnorm(float* resid, const float* delta, int n_parts, in
 }
 
 // ------------------------------------------------------------------ RMSNorm of rows of any width
-// One wave a row.
-template <typename T>
-__global__ void rmsnorm_rows_kernel(const T* __restrict__ x, const void* __restrict__ gain, int gain_is_f32,
-                                    float gain_offset, float eps, T* __restrict__ out, int n_rows, int width) {
+// One wave a row; rows of x may be pieces of longer ones (x_stride values apart).
+template <typename T, typename TOut>
+__global__ void rmsnorm_rows_kernel(const T* __restrict__ x, size_t x_stride, const void* __restrict__ gain, int gain_is_f32,
+                                    float gain_offset, float eps, TOut* __restrict__ out, int n_rows, int width) {
   const int row = blockIdx.x * (blockDim.x / SYN_WAVE) + threadIdx.x / SYN_WAVE;
   if (row >= n_rows) return;
   const int lane = threadIdx.x % SYN_WAVE;
-  const T* xr = x + (size_t)row * width;
-  T* o = out + (size_t)row * width;
+  const T* xr = x + (size_t)row * x_stride;
+  TOut* o = out + (size_t)row * width;
   float ss = 0.f;
   for (int i = lane; i < width; i += SYN_WAVE) {
     float v = to_f32<T>(xr[i]);
@@ -213,20 +213,23 @@ __global__ void rmsnorm_rows_kernel(const T* __restrict__ x, const void* __restr
   ss = wave_sum(ss);
   const float inv = rsqrtf(ss / (float)width + eps);
   for (int i = lane; i < width; i += SYN_WAVE)
-    o[i] = from_f32<T>(load_gain(gain, gain_is_f32, i, gain_offset) * to_f32<T>(xr[i]) * inv);
+    o[i] = from_f32<TOut>(load_gain(gain, gain_is_f32, i, gain_offset) * to_f32<T>(xr[i]) * inv);
 }
 
-SYN_EXPORT int syn_rmsnorm_rows(const void* x, int is_f32, const void* gain, int gain_is_f32, float gain_offset,
-                                float eps, void* out, int n_rows, int width, hipStream_t stream) {
+SYN_EXPORT int syn_rmsnorm_rows(const void* x, int is_f32, long x_stride, const void* gain, int gain_is_f32,
+                                float gain_offset, float eps, void* out, int out_is_f32, int n_rows, int width,
+                                hipStream_t stream) {
   SYN_CHECK(n_rows > 0 && width > 0, "rmsnorm_rows: empty input (%d rows, width %d)", n_rows, width);
+  SYN_CHECK(x_stride >= width && (is_f32 || !out_is_f32), "rmsnorm_rows: rows of %d values %ld apart", width, x_stride);
   const int wpb = 4;
   const int grid = (n_rows + wpb - 1) / wpb;
-  if (is_f32)
-    rmsnorm_rows_kernel<float><<<grid, wpb * SYN_WAVE, 0, stream>>>((const float*)x, gain, gain_is_f32, gain_offset,
-                                                                    eps, (float*)out, n_rows, width);
-  else
-    rmsnorm_rows_kernel<bf16><<<grid, wpb * SYN_WAVE, 0, stream>>>((const bf16*)x, gain, gain_is_f32, gain_offset,
-                                                                   eps, (bf16*)out, n_rows, width);
+#define SYN_RR(TIn, TOut)                                                                                                 \
+  rmsnorm_rows_kernel<TIn, TOut><<<grid, wpb * SYN_WAVE, 0, stream>>>((const TIn*)x, (size_t)x_stride, gain, gain_is_f32, \
+                                                                      gain_offset, eps, (TOut*)out, n_rows, width)
+  if (!is_f32) SYN_RR(bf16, bf16);
+  else if (out_is_f32) SYN_RR(float, float);
+  else SYN_RR(float, bf16);
+#undef SYN_RR
   SYN_LAUNCH_CHECK("rmsnorm_rows");
   return 0;
 }

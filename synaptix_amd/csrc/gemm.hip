@@ -25,12 +25,14 @@
 
 #include "common.h"
 
-// What a kernel does with its 32-bit sums: store them as float or as bf16, or (the kernels over paired
-// gate/up rows) store act(gate) * up as bf16 with the activation `act` of gate_activation.
+// What a kernel does with its 32-bit sums: store them as float or as bf16, behind `point` of point_activation if one is
+// asked for, or (the kernels over paired gate/up rows) store act(gate) * up as bf16 with the activation `act` of
+// gate_activation.
 struct Epilogue {
   int out_is_f32;
   int act;
   float limit;      // the bound of an activation that has one (gated, csrc/common.h)
+  int point;        // SYN_POINT_NONE, or what a plain product's sums pass before they are stored
 };
 
 // ------------------------------------------------------------------ SIMT, any type
@@ -40,7 +42,8 @@ struct Epilogue {
 
 template <typename TIn, typename TOut>
 __global__ void __launch_bounds__(256)
-gemm_simt_kernel(const TIn* __restrict__ x, const TIn* __restrict__ w, TOut* __restrict__ out, int M, int N, int K) {
+gemm_simt_kernel(const TIn* __restrict__ x, const TIn* __restrict__ w, TOut* __restrict__ out, int M, int N, int K,
+                 int point) {
   __shared__ float xs[SIMT_BK][SIMT_BM + 1];
   __shared__ float ws[SIMT_BK][SIMT_BN + 1];
   const int tid = threadIdx.x;
@@ -75,7 +78,7 @@ gemm_simt_kernel(const TIn* __restrict__ x, const TIn* __restrict__ w, TOut* __r
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int gm = m0 + tm + i, gn = n0 + tn + j;
-      if (gm < M && gn < N) out[(size_t)gm * N + gn] = from_f32<TOut>(acc[i][j]);
+      if (gm < M && gn < N) out[(size_t)gm * N + gn] = from_f32<TOut>(point_activation(point, acc[i][j]));
     }
 }
 
@@ -152,7 +155,7 @@ gemm_skinny_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w, void*
       const int t = idx / 256, j = (idx / 64) % 4, ln = idx % 64;
       const int m = 4 * (ln / 16) + j, n = (blockIdx.x * TILES + t) * 16 + ln % 16;
       if (m < M && n < N) {
-        const float v = summed(t, j, ln);
+        const float v = point_activation(ep.point, summed(t, j, ln));
         if (ep.out_is_f32)
           ((float*)out)[(size_t)m * N + n] = v;
         else
@@ -325,6 +328,7 @@ gemm_packed_kernel(const bf16* __restrict__ x, const bf16* __restrict__ wp, void
       if (rn.resid) {   // the same for the whole workgroup
         resid_norm_store(rn, in, m, n, N, v, r0, g0);
       } else if (in) {
+        v = point_activation(ep.point, v);
         if (ep.out_is_f32)
           ((float*)out)[((size_t)blockIdx.y * M + m) * N + n] = v;
         else
@@ -407,6 +411,7 @@ gemm_packed2_kernel(const bf16* __restrict__ x, const bf16* __restrict__ wp, voi
       if (m < M && n < N && (t == 0 || second)) {
         float v = summed(t, j, ln);
         if (rn.ss) v *= inv[m];
+        v = point_activation(ep.point, v);
         if (ep.out_is_f32) ((float*)out)[((size_t)blockIdx.y * M + m) * N + n] = v;
         else ((bf16*)out)[(size_t)m * N + n] = (bf16)v;
       }
@@ -486,10 +491,11 @@ __device__ __forceinline__ void store_tiles(const f32x16 (&acc)[TM][TN], void* _
           const int m = mw + i * 32 + 8 * (e / 4) + 4 * (lane / 32) + e % 4;
           const int n = nw + j * 32 + lane % 32;
           if (m < M && n < N) {
+            const float v = point_activation(ep.point, acc[i][j][e]);
             if (ep.out_is_f32)
-              ((float*)out)[(slice * M + m) * N + n] = acc[i][j][e];
+              ((float*)out)[(slice * M + m) * N + n] = v;
             else
-              ((bf16*)out)[(size_t)m * N + n] = (bf16)acc[i][j][e];
+              ((bf16*)out)[(size_t)m * N + n] = (bf16)v;
           }
         }
   }
@@ -1032,8 +1038,11 @@ static int launch_large(const bf16* x, Weight w, void* out, Epilogue ep, int M, 
 // reader adds the slices.
 // w_packed: w is the weight in fragment order (pack_weight; bf16, N a multiple of 16, K of 128): for the tiles that
 // load straight into LDS; the other kernels read plain rows only.
+// point: what the finished sums pass before they are stored (point_activation; one slice).
 SYN_EXPORT int syn_gemm(const void* x, const void* w, void* out, int dtype, int M, int N, int K, int force_simt,
-                        int slices, int w_packed, hipStream_t stream) {
+                        int slices, int w_packed, int point, hipStream_t stream) {
+  SYN_CHECK(point >= 0 && point < SYN_POINT_COUNT && (point == SYN_POINT_NONE || slices == 1),
+            "gemm: activation code %d over %d slices", point, slices);
   SYN_CHECK(M > 0 && N > 0 && K > 0, "gemm: empty shape M=%d N=%d K=%d", M, N, K);
   SYN_CHECK(!w_packed || (dtype != 0 && !force_simt && N % 16 == 0 && K % 128 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0),
             "gemm: a weight in fragment order needs bf16 operands, N = %d a multiple of 16 and K = %d of 128", N, K);
@@ -1042,19 +1051,20 @@ SYN_EXPORT int syn_gemm(const void* x, const void* w, void* out, int dtype, int 
             "gemm: %d slices of K need bf16 operands and a float output (and beyond 64 rows a K that is a multiple of 64; K = %d)", slices, K);
   const dim3 simt_grid((N + SIMT_BN - 1) / SIMT_BN, (M + SIMT_BM - 1) / SIMT_BM);
   if (dtype == 0) {
-    gemm_simt_kernel<float, float><<<simt_grid, 256, 0, stream>>>((const float*)x, (const float*)w, (float*)out, M, N, K);
+    gemm_simt_kernel<float, float><<<simt_grid, 256, 0, stream>>>((const float*)x, (const float*)w, (float*)out, M, N, K, point);
     SYN_LAUNCH_CHECK("gemm_simt");
     return 0;
   }
   const int out_is_f32 = dtype == 2;
-  const Epilogue ep = {out_is_f32, SYN_ACT_SILU, 0.f};   // (no activation in a plain product)
+  const Epilogue ep = {out_is_f32, SYN_ACT_SILU, 0.f, point};   // (no gate in a plain product)
   const bool aligned = (K % 8 == 0) && ((uintptr_t)x % 16 == 0) && ((uintptr_t)w % 16 == 0);
   SYN_CHECK(slices == 1 || aligned, "gemm: slices of K need 16-byte aligned operands");
   if (force_simt || !aligned) {
     if (out_is_f32)
-      gemm_simt_kernel<bf16, float><<<simt_grid, 256, 0, stream>>>((const bf16*)x, (const bf16*)w, (float*)out, M, N, K);
+      gemm_simt_kernel<bf16, float><<<simt_grid, 256, 0, stream>>>((const bf16*)x, (const bf16*)w, (float*)out, M, N, K,
+                                                                  point);
     else
-      gemm_simt_kernel<bf16, bf16><<<simt_grid, 256, 0, stream>>>((const bf16*)x, (const bf16*)w, (bf16*)out, M, N, K);
+      gemm_simt_kernel<bf16, bf16><<<simt_grid, 256, 0, stream>>>((const bf16*)x, (const bf16*)w, (bf16*)out, M, N, K, point);
     SYN_LAUNCH_CHECK("gemm_simt");
     return 0;
   }
@@ -1122,7 +1132,7 @@ SYN_EXPORT int syn_gemm_swiglu(const void* x, const void* w, void* out, int M, i
   SYN_CHECK(M > 0 && N > 0 && K > 0, "gemm_swiglu: empty shape M=%d N=%d K=%d", M, N, K);
   SYN_CHECK(!w_packed || K % 128 == 0, "gemm_swiglu: a weight in fragment order needs K = %d a multiple of 128", K);
   SYN_CHECK(act >= 0 && act < SYN_ACT_COUNT, "gemm_swiglu: unknown activation code %d", act);
-  const Epilogue ep = {0, act, limit};
+  const Epilogue ep = {0, act, limit, SYN_POINT_NONE};
   SYN_CHECK(N % 32 == 0, "gemm_swiglu: %d paired rows are no multiple of 32", N);
   SYN_CHECK(K % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0,
             "gemm_swiglu: K = %d must be a multiple of 8 and the operands 16-byte aligned", K);
@@ -1165,14 +1175,17 @@ SYN_EXPORT int syn_gemm_swiglu(const void* x, const void* w, void* out, int M, i
 //   ss [M, ss_groups] float (or null): the sums of row m are multiplied by rsqrt(sum(ss[m, :]) / norm_dim + eps);
 //   resid [M, N] float (or null; then float sums, one slice, not paired, `out` unused): resid += sums,
 //   xs [M, N] bf16 = (gain_offset + gain[n]) * resid, ss_out [M, N / 16] = sums of resid^2 over groups of 16 columns.
+// point: as for syn_gemm.
 SYN_EXPORT int syn_gemm_packed_norm(const void* x, const void* wp, void* out, int out_code, int M, int N, int K, int paired,
                                     int act, float limit, int slices, const float* ss, int ss_groups, int norm_dim, float eps,
                                     float* resid, void* xs, float* ss_out, const void* gain, int gain_is_f32,
-                                    float gain_offset, hipStream_t stream) {
+                                    float gain_offset, int point, hipStream_t stream) {
+  SYN_CHECK(point >= 0 && point < SYN_POINT_COUNT && (point == SYN_POINT_NONE || (slices == 1 && !paired && !resid)),
+            "gemm_packed: activation code %d belongs to a plain product in one slice", point);
   SYN_CHECK(act >= 0 && act < SYN_ACT_COUNT, "gemm_packed: unknown activation code %d", act);
   SYN_CHECK(slices >= 1 && slices <= 64 && (slices == 1 || (out_code == 2 && !paired)),
             "gemm_packed: %d slices of K need a float output [slices, M, N] and no activation", slices);
-  const Epilogue ep = {out_code == 2, act, limit};
+  const Epilogue ep = {out_code == 2, act, limit, point};
   SYN_CHECK(M > 0 && M <= 16 && N > 0 && K > 0, "gemm_packed: M = %d (1 .. 16), N = %d, K = %d", M, N, K);
   SYN_CHECK(N % 16 == 0 && K % 32 == 0 && (!paired || N % 32 == 0),
             "gemm_packed: N = %d must be a multiple of 16 (32 for paired rows), K = %d of 32", N, K);
@@ -1210,7 +1223,7 @@ SYN_EXPORT int syn_gemm_packed_norm(const void* x, const void* wp, void* out, in
 }
 
 SYN_EXPORT int syn_gemm_packed(const void* x, const void* wp, void* out, int out_code, int M, int N, int K, int paired,
-                               int act, float limit, int slices, hipStream_t stream) {
+                               int act, float limit, int slices, int point, hipStream_t stream) {
   return syn_gemm_packed_norm(x, wp, out, out_code, M, N, K, paired, act, limit, slices, nullptr, 0, 0, 0.f, nullptr, nullptr,
-                              nullptr, nullptr, 0, 0.f, stream);
+                              nullptr, nullptr, 0, 0.f, point, stream);
 }

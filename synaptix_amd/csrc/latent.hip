@@ -1,7 +1,8 @@
 // Intake of latent attention: what a token's fused projection becomes before its attention runs.
 //
-// proj [N][width] float holds  [ q: heads x (dim | rot_dim) | down: rank + rot_dim | ... ]  (what lies behind, a gate,
-// stays where it is).  For each token at position p:
+// proj [N][width] float holds  [ q: heads x (dim | rot_dim) | ... ], down [N][down_stride] float  [ rank + rot_dim | ... ]:
+// columns of one fused product (what lies behind, a gate, stays where it is), or rows of two products where the queries
+// come through a latent of their own.  For each token at position p:
 //   c      = RMSNorm(down[0 .. rank)) * gain                      the latent that keys and values are made from
 //   k_rot  = rotate(down[rank .. rank + rot_dim), p)               one rotated key part for all heads
 //   q_nope[h] = q[h][0 .. dim)                                     -> q_nope [N][heads][dim]
@@ -23,7 +24,8 @@ __device__ __forceinline__ int latent_v_offset(int d, int slot) {
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-latent_intake_kernel(const float* __restrict__ proj, int width, const void* __restrict__ gain, int gain_is_f32, float eps,
+latent_intake_kernel(const float* __restrict__ proj, int width, const float* __restrict__ down_rows, int down_stride,
+                     const void* __restrict__ gain, int gain_is_f32, float eps,
                      const float* __restrict__ cos_t, const float* __restrict__ sin_t, int n_pairs,
                      T* __restrict__ q_nope, T* __restrict__ q_full, T* __restrict__ k_pages, T* __restrict__ v_pages,
                      const int* __restrict__ page_table, int table_stride, const int* __restrict__ tok_seq,
@@ -50,7 +52,7 @@ latent_intake_kernel(const float* __restrict__ proj, int width, const void* __re
     q_full[((size_t)tok * heads + h) * R + rank + e] = from_f32<T>(v);
   }
   if (!write_kv) return;            // (uniform: no barrier has been reached)
-  const float* down = row + heads * qd;
+  const float* down = down_rows + (size_t)tok * down_stride;
   float ss = 0.f;
   for (int d = threadIdx.x; d < rank; d += blockDim.x) ss += down[d] * down[d];
   ss = block_sum(ss, red);
@@ -74,25 +76,27 @@ latent_intake_kernel(const float* __restrict__ proj, int width, const void* __re
   }
 }
 
-SYN_EXPORT int syn_latent_intake(const float* proj, int width, const void* gain, int gain_is_f32, float eps,
+SYN_EXPORT int syn_latent_intake(const float* proj, int width, const float* down, int down_stride, const void* gain,
+                                 int gain_is_f32, float eps,
                                  const float* cos_t, const float* sin_t, int n_pairs, int capacity, int max_position,
                                  void* q_nope, void* q_full, void* k_pages, void* v_pages, int is_f32,
                                  const int* page_table, int table_stride, const int* tok_seq, const int* tok_pos,
                                  int n_tokens, int heads, int dim, int rot, int rank, int write_kv, int v_fragments,
                                  hipStream_t stream) {
   SYN_CHECK(n_tokens > 0 && heads > 0 && dim > 0 && rot >= 0 && rank > 0, "latent_intake: empty input");
-  SYN_CHECK(width >= heads * (dim + rot) + rank + rot, "latent_intake: rows of %d values do not hold the queries and the latent", width);
+  SYN_CHECK(width >= heads * (dim + rot) && down_stride >= rank + rot,
+            "latent_intake: rows of %d and %d values do not hold the queries and the latent", width, down_stride);
   SYN_CHECK(n_pairs >= 0 && 2 * n_pairs <= rot, "latent_intake: %d rotated pairs in %d values", n_pairs, rot);
   SYN_CHECK(!v_fragments || rank % 16 == 0, "latent_intake: value pages in fragment order need a latent that is a multiple of 16, not %d", rank);
   SYN_CHECK(n_pairs == 0 || (cos_t && sin_t && max_position < capacity),
             "latent_intake: position %d is beyond the rotation's table of %d", max_position, capacity);
   if (is_f32)
-    latent_intake_kernel<float><<<n_tokens, 256, 0, stream>>>(proj, width, gain, gain_is_f32, eps, cos_t, sin_t, n_pairs,
+    latent_intake_kernel<float><<<n_tokens, 256, 0, stream>>>(proj, width, down, down_stride, gain, gain_is_f32, eps, cos_t, sin_t, n_pairs,
                                                               (float*)q_nope, (float*)q_full, (float*)k_pages,
                                                               (float*)v_pages, page_table, table_stride, tok_seq, tok_pos,
                                                               heads, dim, rot, rank, write_kv, v_fragments);
   else
-    latent_intake_kernel<bf16><<<n_tokens, 256, 0, stream>>>(proj, width, gain, gain_is_f32, eps, cos_t, sin_t, n_pairs,
+    latent_intake_kernel<bf16><<<n_tokens, 256, 0, stream>>>(proj, width, down, down_stride, gain, gain_is_f32, eps, cos_t, sin_t, n_pairs,
                                                              (bf16*)q_nope, (bf16*)q_full, (bf16*)k_pages, (bf16*)v_pages,
                                                              page_table, table_stride, tok_seq, tok_pos, heads, dim, rot,
                                                              rank, write_kv, v_fragments);

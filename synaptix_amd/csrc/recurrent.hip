@@ -6,6 +6,7 @@
 //   state_space_scan   a scalar decay a head:   S <- exp(-exp(A) dt) S + dt B x^T,  y = S^T C + D x      (S: N x P)
 //   channel_delta_scan a decay for every key channel and the delta rule:
 //                      S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q                 (S: D x P)
+//   head_delta_scan    the same with one decay a head, S <- g S
 //   diff_heads         two softmax maps over the same values, o = rms_norm(a1 - lambda a2) (1 - c)
 //
 // Everything here is 32-bit FMA: inputs are the float sums of the projections, states are float.  The scans walk a
@@ -319,14 +320,14 @@ SYN_EXPORT int syn_state_space_scan(const float* xbc, const float* dt, int dt_st
   return 0;
 }
 
-// ---------------------------------------------------------------- delta rule with a decay for every key channel
+// ---------------------------------------------------------------- delta rule, a decay for every key channel or one a head
 // qkv [N][(2 K + H E)] float behind the convolution: q (K heads x D), k (K x D), v (H x E); beta: float rows, one a head,
-// before the sigmoid; a: float rows of a_stride values, H * D of them used, before bias and softplus; state
-// [rows][H][D][E]; o [N][H * E] float.
+// before the sigmoid; a: float rows of a_stride values, before bias and softplus, of which H * D are used (CHANNEL: a decay
+// for every key channel) or H (one a head); state [rows][H][D][E]; o [N][H * E] float.
 // Staged for each token: q and k as unit vectors (q also times q_scale), the decays, k . q.
-template <int R, int SL>
+template <int R, int SL, bool CHANNEL>
 __global__ void __launch_bounds__(64 * SL)
-channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict__ beta, int beta_stride,
+delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict__ beta, int beta_stride,
                           const float* __restrict__ a, int a_stride, const float* __restrict__ a_bias,
                           const float* __restrict__ a_log, float q_scale, float unit_eps, float* __restrict__ state,
                           int state_rows, const int* __restrict__ seq_start, const int* __restrict__ seq_slot,
@@ -335,8 +336,8 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
   extern __shared__ __attribute__((aligned(16))) float lds[];
   float* qs = lds;                          // [tb_max][LD]
   float* ks = qs + tb_max * LD;             // [tb_max][LD]
-  float* gs = ks + tb_max * LD;             // [tb_max][LD]
-  float* vs = gs + tb_max * LD;             // [tb_max][64]
+  float* gs = ks + tb_max * LD;             // [tb_max][LD], or [tb_max] with one decay a head
+  float* vs = gs + tb_max * (CHANNEL ? LD : 1);      // [tb_max][64]
   float* kq = vs + tb_max * 64;             // [tb_max]
   float* bt = kq + tb_max;                  // [tb_max]
   const int CB = blockDim.x / SYN_WAVE * (64 / SL);      // columns of this workgroup
@@ -360,7 +361,8 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
   // a chunk's values on their way from memory: a wave stages the tokens wave, wave + n_waves (the host keeps a chunk within
   // RC_TPW tokens a wave), asked for while the chunk before is walked
   constexpr int DL = (SL * R + 63) / 64;
-  float pq[RC_TPW][DL], pk[RC_TPW][DL], pa[RC_TPW][DL], pv[RC_TPW], pbeta[RC_TPW];
+  constexpr int AL = CHANNEL ? DL : 1;
+  float pq[RC_TPW][DL], pk[RC_TPW][DL], pa[RC_TPW][AL], pv[RC_TPW], pbeta[RC_TPW];
   auto fetch = [&](int t0) {
     const int tb = min(tb_max, n_new - t0);
 #pragma unroll
@@ -368,7 +370,9 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
       const int t = wave + j * n_waves;
       pv[j] = pbeta[j] = 0.f;
 #pragma unroll
-      for (int i = 0; i < DL; ++i) pq[j][i] = pk[j][i] = pa[j][i] = 0.f;
+      for (int i = 0; i < DL; ++i) pq[j][i] = pk[j][i] = 0.f;
+#pragma unroll
+      for (int i = 0; i < AL; ++i) pa[j][i] = 0.f;
       if (t < tb) {
         const size_t tok = s0 + t0 + t;
         const float* qr = qkv + tok * width + kvh * D;
@@ -378,9 +382,10 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
           const int d = lane + 64 * i;
           if (d < D) {
             pq[j][i] = qr[d], pk[j][i] = kr[d];
-            pa[j][i] = a[tok * (size_t)a_stride + head * D + d] + a_bias[head * D + d];
+            if constexpr (CHANNEL) pa[j][i] = a[tok * (size_t)a_stride + head * D + d] + a_bias[head * D + d];
           }
         }
+        if constexpr (!CHANNEL) pa[j][0] = a[tok * (size_t)a_stride + head] + a_bias[head];
         if (lane < CB && p0 + lane < E) pv[j] = qkv[tok * width + 2 * K * D + head * E + p0 + lane];
         pbeta[j] = beta[tok * beta_stride + head];
       }
@@ -407,10 +412,11 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
             const int at = t * LD + rc_at(d, R);
             qs[at] = pq[j][i] * iq;
             ks[at] = pk[j][i] * ik;
-            gs[at] = d < D ? expf(A * rc_softplus(pa[j][i])) : 1.f;
+            if constexpr (CHANNEL) gs[at] = d < D ? expf(A * rc_softplus(pa[j][i])) : 1.f;
           }
         }
         if (lane == 0) {
+          if constexpr (!CHANNEL) gs[t] = expf(A * rc_softplus(pa[j][0]));
           kq[t] = dot * iq * ik;
           bt[t] = 1.f / (1.f + expf(-pbeta[j]));
         }
@@ -423,24 +429,43 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
     for (int t = 0; t < tb; ++t) {
       const float4* qt = (const float4*)(qs + t * LD + slice * (R + 4));
       const float4* kt = (const float4*)(ks + t * LD + slice * (R + 4));
-      const float4* gt = (const float4*)(gs + t * LD + slice * (R + 4));
       float rk[4] = {0.f, 0.f, 0.f, 0.f}, rq[4] = {0.f, 0.f, 0.f, 0.f};
+      if constexpr (CHANNEL) {
+        const float4* gt = (const float4*)(gs + t * LD + slice * (R + 4));
 #pragma unroll
-      for (int i = 0; i < R; i += 4) {
-        const float4 gv = gt[i / 4], kv = kt[i / 4], qv = qt[i / 4];
-        s[i] *= gv.x, rk[0] = fmaf(s[i], kv.x, rk[0]), rq[0] = fmaf(s[i], qv.x, rq[0]);
-        s[i + 1] *= gv.y, rk[1] = fmaf(s[i + 1], kv.y, rk[1]), rq[1] = fmaf(s[i + 1], qv.y, rq[1]);
-        s[i + 2] *= gv.z, rk[2] = fmaf(s[i + 2], kv.z, rk[2]), rq[2] = fmaf(s[i + 2], qv.z, rq[2]);
-        s[i + 3] *= gv.w, rk[3] = fmaf(s[i + 3], kv.w, rk[3]), rq[3] = fmaf(s[i + 3], qv.w, rq[3]);
+        for (int i = 0; i < R; i += 4) {
+          const float4 gv = gt[i / 4], kv = kt[i / 4], qv = qt[i / 4];
+          s[i] *= gv.x, rk[0] = fmaf(s[i], kv.x, rk[0]), rq[0] = fmaf(s[i], qv.x, rq[0]);
+          s[i + 1] *= gv.y, rk[1] = fmaf(s[i + 1], kv.y, rk[1]), rq[1] = fmaf(s[i + 1], qv.y, rq[1]);
+          s[i + 2] *= gv.z, rk[2] = fmaf(s[i + 2], kv.z, rk[2]), rq[2] = fmaf(s[i + 2], qv.z, rq[2]);
+          s[i + 3] *= gv.w, rk[3] = fmaf(s[i + 3], kv.w, rk[3]), rq[3] = fmaf(s[i + 3], qv.w, rq[3]);
+        }
+      } else {
+        // one decay for the whole state: it multiplies the sums over the old state instead, (g S)^T k = g (S^T k)
+#pragma unroll
+        for (int i = 0; i < R; i += 4) {
+          const float4 kv = kt[i / 4], qv = qt[i / 4];
+          rk[0] = fmaf(s[i], kv.x, rk[0]), rq[0] = fmaf(s[i], qv.x, rq[0]);
+          rk[1] = fmaf(s[i + 1], kv.y, rk[1]), rq[1] = fmaf(s[i + 1], qv.y, rq[1]);
+          rk[2] = fmaf(s[i + 2], kv.z, rk[2]), rq[2] = fmaf(s[i + 2], qv.z, rq[2]);
+          rk[3] = fmaf(s[i + 3], kv.w, rk[3]), rq[3] = fmaf(s[i + 3], qv.w, rq[3]);
+        }
       }
-      const float rks = rc_sum_slices<SL>((rk[0] + rk[1]) + (rk[2] + rk[3]));
-      const float rqs = rc_sum_slices<SL>((rq[0] + rq[1]) + (rq[2] + rq[3]));
+      float rks = rc_sum_slices<SL>((rk[0] + rk[1]) + (rk[2] + rk[3]));
+      float rqs = rc_sum_slices<SL>((rq[0] + rq[1]) + (rq[2] + rq[3]));
+      float g = 1.f;
+      if constexpr (!CHANNEL) g = gs[t], rks *= g, rqs *= g;
       const float u = bt[t] * (vs[t * 64 + mine] - rks);
 #pragma unroll
       for (int i = 0; i < R; i += 4) {
         const float4 kv = kt[i / 4];
-        s[i] = fmaf(kv.x, u, s[i]), s[i + 1] = fmaf(kv.y, u, s[i + 1]);
-        s[i + 2] = fmaf(kv.z, u, s[i + 2]), s[i + 3] = fmaf(kv.w, u, s[i + 3]);
+        if constexpr (CHANNEL) {
+          s[i] = fmaf(kv.x, u, s[i]), s[i + 1] = fmaf(kv.y, u, s[i + 1]);
+          s[i + 2] = fmaf(kv.z, u, s[i + 2]), s[i + 3] = fmaf(kv.w, u, s[i + 3]);
+        } else {
+          s[i] = fmaf(kv.x, u, g * s[i]), s[i + 1] = fmaf(kv.y, u, g * s[i + 1]);
+          s[i + 2] = fmaf(kv.z, u, g * s[i + 2]), s[i + 3] = fmaf(kv.w, u, g * s[i + 3]);
+        }
       }
       // the read-out sees this token's write: (S + k u^T)^T q = S^T q + u (k . q)
       if (slice == 0 && col_ok) o[(size_t)(s0 + t0 + t) * H * E + head * E + p] = fmaf(u, kq[t], rqs);
@@ -453,25 +478,26 @@ channel_delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict
   }
 }
 
-SYN_EXPORT int syn_channel_delta_scan(const float* qkv, const float* beta, int beta_stride, const float* a, int a_stride,
-                                      const float* a_bias, const float* a_log, float q_scale, float unit_eps, float* state,
-                                      int state_rows, const int* seq_start, const int* seq_slot, int n_seqs, int longest,
-                                      float* o, int H, int K, int D, int E, hipStream_t stream) {
-  SYN_CHECK(n_seqs > 0 && longest > 0 && H > 0 && K > 0 && D > 0 && E > 0, "channel_delta_scan: empty input");
-  SYN_CHECK(H % K == 0, "channel_delta_scan: %d heads do not divide into %d key heads", H, K);
-  SYN_CHECK(D <= RC_ROWS_MAX, "channel_delta_scan: keys of %d values (at most %d)", D, RC_ROWS_MAX);
-  SYN_CHECK(beta_stride >= H && state_rows > 0, "channel_delta_scan: rows of %d values for %d heads", beta_stride, H);
-  SYN_CHECK(a_stride >= H * D, "channel_delta_scan: decay rows of %d values for %d heads of %d", a_stride, H, D);
+template <bool CHANNEL>
+static int delta_scan(const char* name, const float* qkv, const float* beta, int beta_stride, const float* a, int a_stride,
+                      const float* a_bias, const float* a_log, float q_scale, float unit_eps, float* state, int state_rows,
+                      const int* seq_start, const int* seq_slot, int n_seqs, int longest, float* o, int H, int K, int D, int E,
+                      hipStream_t stream) {
+  SYN_CHECK(n_seqs > 0 && longest > 0 && H > 0 && K > 0 && D > 0 && E > 0, "%s: empty input", name);
+  SYN_CHECK(H % K == 0, "%s: %d heads do not divide into %d key heads", name, H, K);
+  SYN_CHECK(D <= RC_ROWS_MAX, "%s: keys of %d values (at most %d)", name, D, RC_ROWS_MAX);
+  SYN_CHECK(beta_stride >= H && state_rows > 0, "%s: rows of %d values for %d heads", name, beta_stride, H);
+  SYN_CHECK(a_stride >= (CHANNEL ? H * D : H), "%s: decay rows of %d values for %d heads of %d", name, a_stride, H, D);
   // (always 64 columns a workgroup: staging a token here means norms and decays, which workgroups that split a head's
   // columns would each do again; measured at 32 heads over 2,048 tokens: 1.18 ms with 64 columns, 1.46 ms with 16)
   const int block_cols = 64;
 #define SYN_CD(R, SL)                                                                                                   \
   do {                                                                                                                  \
-    const int per_token = (3 * RC_LD(R, SL) + 64 + 2) * (int)sizeof(float);                                             \
+    const int per_token = ((CHANNEL ? 3 : 2) * RC_LD(R, SL) + 64 + (CHANNEL ? 2 : 3)) * (int)sizeof(float);             \
     const int waves = (min(E, block_cols) + 64 / SL - 1) / (64 / SL), cb = waves * (64 / SL);                           \
     const dim3 grid(H, n_seqs, (E + cb - 1) / cb);                                                                      \
     const int tb = max(1, min(min(min(RC_TB, longest), RC_LDS_BUDGET / per_token), RC_TPW * waves));                    \
-    channel_delta_scan_kernel<R, SL><<<grid, waves * SYN_WAVE, (size_t)tb * per_token, stream>>>(                       \
+    delta_scan_kernel<R, SL, CHANNEL><<<grid, waves * SYN_WAVE, (size_t)tb * per_token, stream>>>(                      \
         qkv, beta, beta_stride, a, a_stride, a_bias, a_log, q_scale, unit_eps, state, state_rows, seq_start, seq_slot,  \
         o, H, K, D, E, tb);                                                                                             \
   } while (0)
@@ -486,8 +512,24 @@ SYN_EXPORT int syn_channel_delta_scan(const float* qkv, const float* beta, int b
     else SYN_CD(16, 16);
   }
 #undef SYN_CD
-  SYN_LAUNCH_CHECK("channel_delta_scan");
+  SYN_LAUNCH_CHECK(name);
   return 0;
+}
+
+SYN_EXPORT int syn_channel_delta_scan(const float* qkv, const float* beta, int beta_stride, const float* a, int a_stride,
+                                      const float* a_bias, const float* a_log, float q_scale, float unit_eps, float* state,
+                                      int state_rows, const int* seq_start, const int* seq_slot, int n_seqs, int longest,
+                                      float* o, int H, int K, int D, int E, hipStream_t stream) {
+  return delta_scan<true>("channel_delta_scan", qkv, beta, beta_stride, a, a_stride, a_bias, a_log, q_scale, unit_eps, state,
+                          state_rows, seq_start, seq_slot, n_seqs, longest, o, H, K, D, E, stream);
+}
+
+SYN_EXPORT int syn_head_delta_scan(const float* qkv, const float* beta, int beta_stride, const float* a, int a_stride,
+                                   const float* a_bias, const float* a_log, float q_scale, float unit_eps, float* state,
+                                   int state_rows, const int* seq_start, const int* seq_slot, int n_seqs, int longest,
+                                   float* o, int H, int K, int D, int E, hipStream_t stream) {
+  return delta_scan<false>("head_delta_scan", qkv, beta, beta_stride, a, a_stride, a_bias, a_log, q_scale, unit_eps, state,
+                           state_rows, seq_start, seq_slot, n_seqs, longest, o, H, K, D, E, stream);
 }
 
 // ---------------------------------------------------------------- two softmax maps over the same values

@@ -204,13 +204,18 @@ def add_rmsnorm(resid, delta, gain, eps, out, rows=None, gain_offset=0.0):
 
 
 def rmsnorm_rows(x, gain, eps, out, gain_offset=0.0):
-    """out = RMSNorm(x) * (gain_offset + gain) over the last axis; x [..., D] bf16|f32, out like x."""
-    _need(x, "rmsnorm_rows.x", (_BF16, _F32))
+    """out = RMSNorm(x) * (gain_offset + gain) over the last axis; x [..., D] bf16|f32, out like x.  A float matrix x may be
+    the first columns of longer rows (columns of a fused projection), and its out may be bf16."""
     D = x.shape[-1]
+    stride = D
+    if isinstance(x, torch.Tensor) and x.dim() == 2 and x.dtype == _F32:
+        stride = _float_rows_view(x, "rmsnorm_rows.x", x.shape[0], D)
+    else:
+        _need(x, "rmsnorm_rows.x", (_BF16, _F32))
     _need(gain, "rmsnorm_rows.gain", (_BF16, _F32), (D,))
-    _need(out, "rmsnorm_rows.out", x.dtype, tuple(x.shape))
-    _call(load_library("core"), "syn_rmsnorm_rows", _ptr(x), _is_f32(x), _ptr(gain), _is_f32(gain),
-          ctypes.c_float(gain_offset), ctypes.c_float(eps), _ptr(out), x.numel() // D, D, _stream())
+    _need(out, "rmsnorm_rows.out", (_BF16, _F32) if x.dtype == _F32 else x.dtype, tuple(x.shape))
+    _call(load_library("core"), "syn_rmsnorm_rows", _ptr(x), _is_f32(x), ctypes.c_long(stride), _ptr(gain), _is_f32(gain),
+          ctypes.c_float(gain_offset), ctypes.c_float(eps), _ptr(out), _is_f32(out), x.numel() // D, D, _stream())
 
 
 def swiglu(gate_up, out, activation="silu"):
@@ -232,13 +237,28 @@ def _packed_shape(w, name, K):
     return w.shape[0] * 16
 
 
-def gemm(x, w, out, force_simt=False):
+# What the sums of a plain product may pass before they are stored (point_activation in csrc/common.h): the activation of an
+# ungated feed-forward.  "relu_squared": max(z, 0)^2
+POINT_ACTIVATIONS = {"relu_squared": 1}
+
+
+def point_code(name) -> int:
+    if name is None:
+        return 0
+    if name not in POINT_ACTIVATIONS:
+        raise KernelError(f"activation {name!r}: the plain products apply {sorted(POINT_ACTIVATIONS)}")
+    return POINT_ACTIVATIONS[name]
+
+
+def gemm(x, w, out, force_simt=False, point=None):
     """out[M, N] = x[M, K] . w[N, K]^T with 32-bit accumulation.
     float x float -> float (plain FMA); bf16 x bf16 -> bf16 or float (MFMA).
     A float out of shape [S, M, N] (bf16 operands) receives S partial sums over slices of K
     instead; their sum over S is the product.
     w may be the weight in fragment order (pack_weight: four dimensions): the tiles for 9 rows and more read it
-    where K is a multiple of 128; for other K the product runs in blocks of 16 rows through gemm_packed."""
+    where K is a multiple of 128; for other K the product runs in blocks of 16 rows through gemm_packed.
+    point: a name of POINT_ACTIVATIONS, applied to the finished sums before they are stored (not to partial sums)."""
+    point_of = point_code(point)
     _need(x, "gemm.x", (_BF16, _F32), (None, None))
     M, K = x.shape
     packed = isinstance(w, torch.Tensor) and w.dim() == 4
@@ -251,7 +271,7 @@ def gemm(x, w, out, force_simt=False):
                 raise KernelError(f"gemm: no slices of K = {K} over a weight in fragment order")
             rows = out[0] if out.dim() == 3 else out
             for m0 in range(0, M, PACKED_BLOCK_ROWS):
-                gemm_packed(x[m0:m0 + PACKED_BLOCK_ROWS], w, rows[m0:m0 + PACKED_BLOCK_ROWS])
+                gemm_packed(x[m0:m0 + PACKED_BLOCK_ROWS], w, rows[m0:m0 + PACKED_BLOCK_ROWS], point=point)
             return
     else:
         _need(w, "gemm.w", x.dtype, (None, K))
@@ -271,7 +291,7 @@ def gemm(x, w, out, force_simt=False):
         _need(out, "gemm.out", (_BF16, _F32), (M, N))
         code = 2 if out.dtype == _F32 else 1
     _call(load_library("core"), "syn_gemm", _ptr(x), _ptr(w), _ptr(out), code, M, N, K, 1 if force_simt else 0,
-          slices, 1 if packed else 0, _stream())
+          slices, 1 if packed else 0, point_of, _stream())
 
 
 PAIR = 16   # rows of the gate and of the up projection alternate in turns of this many
@@ -337,7 +357,7 @@ def unpack_weight(wp):
     return wp.view(nt, nks, 4, 16, 8).permute(0, 3, 1, 2, 4).reshape(nt * 16, nks * 32).contiguous()
 
 
-def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, resid_norm=None):
+def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, resid_norm=None, point=None):
     """out[M, N] (bf16 or float) = x[M, K] . W^T for M <= 16 with wp = pack_weight(W); paired: W holds gate and
     up rows in turns of 16 (pair_rows) and out [M, N / 2] bf16 = act(gate) * up.  A float out of shape
     [S, M, N] receives S partial sums over slices of K instead.
@@ -346,7 +366,9 @@ def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, res
     resid_norm = (resid [M, N] float, gain [N], gain_offset, xs [M, N] bf16, ss [M, N / 16] float) with out None:
     the sums are added into resid, xs = (gain_offset + gain) * resid, ss = sums of resid^2 over groups of 16 columns;
     row_scale = (ss [M, G] float, dim, eps): the sums of row m are multiplied by rsqrt(sum(ss[m]) / dim + eps), which
-    makes this the product over the normed rows when x is the xs that came with ss."""
+    makes this the product over the normed rows when x is the xs that came with ss.
+    point: as for gemm (behind the row's factor)."""
+    point_of = point_code(point)
     _need(x, "gemm_packed.x", _BF16, (None, None))
     M, K = x.shape
     if K % 32:
@@ -386,12 +408,12 @@ def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, res
         out_code = 2 if out.dtype == _F32 else 1
     if row_scale is None and resid_norm is None:
         _call(load_library("core"), "syn_gemm_packed", _ptr(x), _ptr(wp), _ptr(out), out_code,
-              M, N, K, 1 if paired else 0, *_activation_args(activation), slices, _stream())
+              M, N, K, 1 if paired else 0, *_activation_args(activation), slices, point_of, _stream())
         return
     _call(load_library("core"), "syn_gemm_packed_norm", _ptr(x), _ptr(wp), _ptr(out), out_code, M, N, K,
           1 if paired else 0, *_activation_args(activation), slices, _ptr(ss), int(groups), int(dim), ctypes.c_float(eps),
           _ptr(resid), _ptr(xs), _ptr(ss_out), _ptr(gain), _is_f32(gain) if gain is not None else 0,
-          ctypes.c_float(gain_offset), _stream())
+          ctypes.c_float(gain_offset), point_of, _stream())
 
 
 _compute_units = None
@@ -822,7 +844,8 @@ def _check_window_pages(k_pages, v_pages, dtype, nkv, dim, vdim, name, v_share=1
 
 
 def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_pos, q_gain, k_gain, eps,
-                  n_heads, n_kv_heads, dim, vdim, write_kv=True, rotation=None, v_share=1, pairs=False):
+                  n_heads, n_kv_heads, dim, vdim, write_kv=True, rotation=None, v_share=1, pairs=False,
+                  norm_whole=False, values_are_keys=False, q_temp=None):
     """proj [N, width] float: the fused projection [q | k | v | ...]; bias float [>= q, k, v columns] or None.  q and k
     heads get their bias and (with gains, float [dim]) an RMSNorm over the head; q goes to q_out [N, nh * dim], k and v
     (with its bias) into the pages of sequence tok_seq[n] at position tok_pos[n].
@@ -830,14 +853,22 @@ def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_
     the angles of the token's position, value i paired with value i + rot / 2 (the caller sees to it that the tables
     reach the step's last position); with `pairs` value 2 i is paired with value 2 i + 1.  v_share: there are
     nkv / v_share value heads (and rows of v in proj).  write_kv False: the pages are another layer's and are left
-    alone; proj and bias then need to hold the queries only."""
+    alone; proj and bias then need to hold the queries only.  norm_whole: the norms run over all query heads at once and
+    over all key heads at once, with gains [nh * dim] and [nkv * dim].  values_are_keys: proj has no v columns, the values
+    are the keys as projected (with their bias, before norm and rotation).  q_temp = (coef, every): queries at position p
+    are multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
     nh, nkv = n_heads, n_kv_heads
     _need(proj, "window_intake.proj", _F32, (None, None))
     N, width = proj.shape
     if v_share < 1 or nkv % v_share:
         raise KernelError(f"window_intake: {nkv} kv heads in shares of {v_share} value heads")
     nv = nkv // v_share
-    used = (nh + nkv) * dim + nv * vdim if write_kv else nh * dim
+    if values_are_keys and (v_share != 1 or vdim != dim):
+        raise KernelError(f"window_intake: values of {vdim} that are keys of {dim}")
+    used = (nh + nkv) * dim + (0 if values_are_keys else nv * vdim) if write_kv else nh * dim
+    coef, every = (float(q_temp[0]), int(q_temp[1])) if q_temp is not None else (0.0, 1)
+    if every <= 0:
+        raise KernelError(f"window_intake: a temperature that steps every {every} positions")
     if width < used:
         raise KernelError(f"window_intake: rows of {width} values do not hold {'q, k and v' if write_kv else 'q'} ({used})")
     if bias is not None:
@@ -861,12 +892,15 @@ def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_
     if (q_gain is None) != (k_gain is None):
         raise KernelError("window_intake: q and k gains come together")
     if q_gain is not None:
-        _need(q_gain, "window_intake.q_gain", _F32, (dim,))
-        _need(k_gain, "window_intake.k_gain", _F32, (dim,))
+        _need(q_gain, "window_intake.q_gain", _F32, (nh * dim if norm_whole else dim,))
+        _need(k_gain, "window_intake.k_gain", _F32, (nkv * dim if norm_whole else dim,))
+    elif norm_whole:
+        raise KernelError("window_intake: a norm over all heads without its gains")
     _call(load_library("core"), "syn_window_intake", _ptr(proj), width, _ptr(bias), _ptr(q_out), _ptr(k_pages),
           _ptr(v_pages), _is_f32(q_out), _ptr(page_table), page_table.shape[1], _ptr(tok_seq), _ptr(tok_pos),
           _ptr(q_gain), _ptr(k_gain), ctypes.c_float(eps), _ptr(cos), _ptr(sin), rot, 1 if pairs else 0, N, nh, nkv, nv,
-          dim, vdim, 1 if write_kv else 0, _stream())
+          dim, vdim, 1 if write_kv else 0, 1 if norm_whole else 0, 1 if values_are_keys else 0, ctypes.c_float(coef), every,
+          _stream())
 
 
 def window_attention(q, k_pages, v_pages, page_table, tok_seq, tok_pos, out, scale, n_heads, n_kv_heads, dim, vdim,
@@ -1026,10 +1060,13 @@ def matrix_memory_scan(proj, i_bias, f_bias, gate_cap, q_scale, state, seq_start
           _ptr(seq_slot), B, _ptr(out), H, dim, vdim, 1 if chunked else 0, N, _ptr(work), _stream())
 
 
-def head_norm_gate(o, gain, eps, gate, out, n_heads, vdim, silu_first=False):
+def head_norm_gate(o, gain, eps, gate, out, n_heads, vdim, silu_first=False, silu=False):
     """out[n, h] = o[n, h] / rms(o[n, h]) * gain[h] * sigmoid(gate[n, h]): o [N, H * vdim] float, gain float [H * vdim]
     or None, gate a float view [N, >= H * vdim] (see _float_rows_view) or None, out [N, H * vdim] bf16 or float.
-    silu_first: the gate comes before the norm, x = o * silu(gate), out = x / rms(x) * gain."""
+    silu_first: the gate comes before the norm, x = o * silu(gate), out = x / rms(x) * gain; silu: behind it, but as
+    silu(gate) instead of sigmoid(gate)."""
+    if silu_first and silu:
+        raise KernelError("head_norm_gate: the gate acts before the norm or behind it")
     _need(o, "head_norm_gate.o", _F32, (None, n_heads * vdim))
     N = o.shape[0]
     if gain is not None:
@@ -1037,7 +1074,7 @@ def head_norm_gate(o, gain, eps, gate, out, n_heads, vdim, silu_first=False):
     stride = _float_rows_view(gate, "head_norm_gate.gate", N, n_heads * vdim) if gate is not None else 0
     _need(out, "head_norm_gate.out", (_BF16, _F32), (N, n_heads * vdim))
     _call(load_library("core"), "syn_head_norm_gate", _ptr(o), _ptr(gain), ctypes.c_float(eps), _ptr(gate), stride,
-          _ptr(out), _is_f32(out), N, n_heads, vdim, 1 if silu_first else 0, _stream())
+          _ptr(out), _is_f32(out), N, n_heads, vdim, 1 if silu_first else (2 if silu else 0), _stream())
 
 
 # ----------------------------------------------------------------------------- short convolutions and scans over a state
@@ -1106,6 +1143,27 @@ def state_space_scan(xbc, dt, dt_bias, a_log, d_skip, state, seq_start, seq_slot
           _ptr(out), H, vdim, n_state, G, _stream())
 
 
+def _delta_scan(name, qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads, n_key_heads,
+                dim, vdim, n_decays, single_tokens):
+    H, K = n_heads, n_key_heads
+    if K <= 0 or H % K:
+        raise KernelError(f"{name}: {H} heads do not divide into {K} key heads")
+    if dim > SCAN_MAX_ROWS:
+        raise KernelError(f"{name}: keys of {dim} values (at most {SCAN_MAX_ROWS})")
+    _need(qkv, name + ".qkv", _F32, (None, 2 * K * dim + H * vdim))
+    N = qkv.shape[0]
+    stride = _float_rows_view(beta, name + ".beta", N, H)
+    a_stride = _float_rows_view(a, name + ".a", N, n_decays)
+    _need(a_bias, name + ".a_bias", _F32, (n_decays,))
+    _need(a_log, name + ".a_log", _F32, (H,))
+    _need(state, name + ".state", _F32, (None, H, dim, vdim))
+    B = _step_seqs(name, seq_start, seq_slot)
+    _need(out, name + ".out", _F32, (N, H * vdim))
+    _call(load_library("core"), "syn_" + name, _ptr(qkv), _ptr(beta), stride, _ptr(a), a_stride, _ptr(a_bias),
+          _ptr(a_log), ctypes.c_float(q_scale), ctypes.c_float(unit_eps), _ptr(state), state.shape[0], _ptr(seq_start),
+          _ptr(seq_slot), B, 1 if single_tokens else max(N, 2), _ptr(out), H, K, dim, vdim, _stream())
+
+
 def channel_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads,
                        n_key_heads, dim, vdim, single_tokens=False):
     """The delta rule with a decay for every key channel over the new tokens of every sequence of the step, in order.
@@ -1116,24 +1174,15 @@ def channel_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, se
     float view [N, >= H]; a a float view [N, >= H * dim]; a_bias float [H * dim]; a_log float [H]; state float
     [rows, H, dim, vdim] (row seq_slot[b]; a negative slot: the last row); out float [N, H * vdim].
     single_tokens: as for state_space_scan."""
-    H, K = n_heads, n_key_heads
-    if K <= 0 or H % K:
-        raise KernelError(f"channel_delta_scan: {H} heads do not divide into {K} key heads")
-    if dim > SCAN_MAX_ROWS:
-        raise KernelError(f"channel_delta_scan: keys of {dim} values (at most {SCAN_MAX_ROWS})")
-    _need(qkv, "channel_delta_scan.qkv", _F32, (None, 2 * K * dim + H * vdim))
-    N = qkv.shape[0]
-    stride = _float_rows_view(beta, "channel_delta_scan.beta", N, H)
-    a_stride = _float_rows_view(a, "channel_delta_scan.a", N, H * dim)
-    _need(a_bias, "channel_delta_scan.a_bias", _F32, (H * dim,))
-    _need(a_log, "channel_delta_scan.a_log", _F32, (H,))
-    _need(state, "channel_delta_scan.state", _F32, (None, H, dim, vdim))
-    B = _step_seqs("channel_delta_scan", seq_start, seq_slot)
-    _need(out, "channel_delta_scan.out", _F32, (N, H * vdim))
-    _call(load_library("core"), "syn_channel_delta_scan", _ptr(qkv), _ptr(beta), stride, _ptr(a), a_stride, _ptr(a_bias),
-          _ptr(a_log),
-          ctypes.c_float(q_scale), ctypes.c_float(unit_eps), _ptr(state), state.shape[0], _ptr(seq_start), _ptr(seq_slot), B,
-          1 if single_tokens else max(N, 2), _ptr(out), H, K, dim, vdim, _stream())
+    _delta_scan("channel_delta_scan", qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads,
+                n_key_heads, dim, vdim, n_heads * dim, single_tokens)
+
+
+def head_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads, n_key_heads,
+                    dim, vdim, single_tokens=False):
+    """channel_delta_scan with one decay a head: a a float view [N, >= H], a_bias float [H], S <- g S."""
+    _delta_scan("head_delta_scan", qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads,
+                n_key_heads, dim, vdim, n_heads, single_tokens)
 
 
 def diff_heads(a, out, lam, eps, post, n_kv_heads, heads_per_kv, vdim):
@@ -1444,18 +1493,25 @@ def latent_v_pages_to_kernel_order(v):
 
 
 def latent_intake(proj, gain, eps, cos, sin, q_nope, q_full, k_pages, v_pages, page_table, tok_seq, tok_pos,
-                  n_heads, dim, rot_dim, rank, max_position, write_kv=True, v_fragments=False):
+                  n_heads, dim, rot_dim, rank, max_position, write_kv=True, v_fragments=False, down=None):
     """From the fused projection proj [N, >= heads * (dim + rot_dim) + rank + rot_dim] float: q_nope [N, heads * dim];
     the rotated query parts into q_full [N, heads * (rank + rot_dim)] behind each head's first `rank` places; the
     token's cache row [RMSNorm(latent) * gain | rotated key part] into k_pages [pages, 1, 64, rank + rot_dim] and the
     normed latent as its value into v_pages [pages, 1, rank, 64].  cos, sin [capacity, pairs]: pairs (2i, 2i + 1) of
     the rotated parts are turned, what lies behind 2 * pairs passes.  v_fragments: the value pages are kept in the order
-    of the bf16 attention kernel's fragments (what latent_attention reads when it runs in tiles)."""
+    of the bf16 attention kernel's fragments (what latent_attention reads when it runs in tiles).
+    down: where the latent and the rotated key part come from another product than the queries (queries that pass a latent
+    of their own): a float view [N, >= rank + rot_dim]; proj then needs to hold the queries only."""
     _need(proj, "latent_intake.proj", _F32, (None, None))
     N, width = proj.shape
-    R = rank + rot_dim
-    if width < n_heads * (dim + rot_dim) + R:
-        raise KernelError(f"latent_intake: rows of {width} values do not hold {n_heads} queries and the latent")
+    R, nq = rank + rot_dim, n_heads * (dim + rot_dim)
+    if down is None:
+        if width < nq + R:
+            raise KernelError(f"latent_intake: rows of {width} values do not hold {n_heads} queries and the latent")
+        down = proj[:, nq:]
+    elif width < nq:
+        raise KernelError(f"latent_intake: rows of {width} values do not hold {n_heads} queries")
+    down_stride = _float_rows_view(down, "latent_intake.down", N, R)
     _need(gain, "latent_intake.gain", (_BF16, _F32), (rank,))
     n_pairs, capacity = 0, 0
     if cos is not None:
@@ -1471,7 +1527,7 @@ def latent_intake(proj, gain, eps, cos, sin, q_nope, q_full, k_pages, v_pages, p
     _need(page_table, "latent_intake.page_table", _I32, (None, None))
     _need(tok_seq, "latent_intake.tok_seq", _I32, (N,))
     _need(tok_pos, "latent_intake.tok_pos", _I32, (N,))
-    _call(load_library("core"), "syn_latent_intake", _ptr(proj), width, _ptr(gain), _is_f32(gain), ctypes.c_float(eps),
+    _call(load_library("core"), "syn_latent_intake", _ptr(proj), width, _ptr(down), down_stride, _ptr(gain), _is_f32(gain), ctypes.c_float(eps),
           _ptr(cos), _ptr(sin), n_pairs, capacity, int(max_position), _ptr(q_nope), _ptr(q_full), _ptr(k_pages),
           _ptr(v_pages), _is_f32(q_nope), _ptr(page_table), page_table.shape[1], _ptr(tok_seq), _ptr(tok_pos), N, n_heads,
           dim, rot_dim, rank, int(bool(write_kv)), int(bool(v_fragments)), _stream())

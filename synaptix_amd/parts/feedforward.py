@@ -72,6 +72,36 @@ class GatedMlp(FeedForward):
         return deferred_product(m, self.w_down)
 
 
+class UngatedMlp(FeedForward):
+    """down( act(up(h)) ), dense: the activation is the first product's epilogue (ops.POINT_ACTIVATIONS).
+    Tensors: prefix + "up" [ff, hidden], "down" [hidden, ff]; `names` renames them."""
+    takes_scaled_rows = True
+    capturable = True
+
+    NAMES = ("up", "down")
+
+    def __init__(self, prefix: str, hidden: int, intermediate: int, activation: str = "relu_squared", names=None):
+        self.names = tuple(names or self.NAMES)
+        try:
+            ops.point_code(activation)
+        except ops.KernelError as e:
+            raise ValueError(f"{prefix}: {e}") from None
+        self.prefix, self.hidden, self.intermediate, self.activation = prefix, hidden, intermediate, activation
+        self.w_up = self.w_down = None
+
+    def tensor_specs(self):
+        p, (up, down) = self.prefix, self.names
+        return {p + up: TensorSpec((self.intermediate, self.hidden)), p + down: TensorSpec((self.hidden, self.intermediate))}
+
+    def load(self, get):
+        # (in fragment order only where the tiles for many rows read that order too)
+        up, down = (get(self.prefix + n) for n in self.names)
+        self.w_up, self.w_down = (Matrix(w, keep_rows=w.shape[1] % 128 != 0) for w in (up, down))
+
+    def forward(self, h, ctx):
+        return deferred_product(linear(h, self.w_up, h.dtype, point=self.activation), self.w_down)
+
+
 class RoutedExperts(FeedForward):
     """A mixture of small experts: each token goes through `top` of them, chosen by a router, and gets the weighted sum
     of their results.

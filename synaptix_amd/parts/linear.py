@@ -182,15 +182,16 @@ def deferred_product(x, w):
     return linear_for_sum(x, w)
 
 
-def linear(x, w, out_dtype):
-    """x [M, K] in the activation type, w a Matrix [N, K]; a weight kept in 32-bit takes the 32-bit product."""
+def linear(x, w, out_dtype, point=None):
+    """x [M, K] in the activation type, w a Matrix [N, K]; a weight kept in 32-bit takes the 32-bit product.
+    point: an activation that the product applies to its sums before it stores them (ops.POINT_ACTIVATIONS)."""
     w = _matrix(w)
     if _use_packed(x, w) and out_dtype in (torch.bfloat16, torch.float32):
         out = torch.empty((x.shape[0], w.shape[0]), dtype=out_dtype, device=x.device)
         if isinstance(x, ScaledRows):
-            ops.gemm_packed(x.rows, w.packed, out, row_scale=x.row_scale)
+            ops.gemm_packed(x.rows, w.packed, out, row_scale=x.row_scale, point=point)
         else:
-            ops.gemm_packed(x, w.packed, out)
+            ops.gemm_packed(x, w.packed, out, point=point)
         return out
     x = as_rows(x)
     if w.dtype != x.dtype:
@@ -200,7 +201,7 @@ def linear(x, w, out_dtype):
             raise TypeError(f"linear: activation {x.dtype} with weight {w.dtype}")
     out = torch.empty((x.shape[0], w.shape[0]), dtype=torch.float32 if x.dtype == torch.float32 else out_dtype,
                       device=x.device)
-    ops.gemm(x, w.data, out)
+    ops.gemm(x, w.data, out, point=point)
     return out if out.dtype == out_dtype else out.to(out_dtype)
 
 

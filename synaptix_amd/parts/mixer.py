@@ -214,6 +214,10 @@ class GatedWindowAttention(Mixer):
     that layer wrote it, with its own queries, mask, sink and gate.  `cache_window`: what the cache keeps where that is
     more than this layer's own mask needs (the layers that share a cache name the same).
 
+    `qk_norm_whole`: the q and k norms run over all heads' values at once (gains of heads x dim and kv heads x dim) instead
+    of head by head.  `values_are_keys`: there is no v tensor; the values are the keys as projected, before norm and
+    rotation.  `q_temp` = (coef, every): the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1).
+
     Tensor names: prefix + "q", "k", "v", "o" (+ ".b" for their biases), "q.norm", "k.norm", "g", "sink"; `names`
     renames them.
     """
@@ -230,7 +234,8 @@ class GatedWindowAttention(Mixer):
                  position: Position | None = None, qk_norm_eps: float | None = None, scale: float | None = None,
                  window: int | None = None, keep_first: int = 0, sink_one: bool = False, bias: bool = False,
                  out_bias: bool = False, gate=False, score_softcap: float | None = None, names: dict | None = None,
-                 chunk: int | None = None, sink: bool = False, shared_kv: bool = False, cache_window=_UNSET):
+                 chunk: int | None = None, sink: bool = False, shared_kv: bool = False, cache_window=_UNSET,
+                 qk_norm_whole: bool = False, values_are_keys: bool = False, q_temp: tuple | None = None):
         if n_kv_heads <= 0 or n_heads % n_kv_heads:
             raise ValueError(f"{n_heads} heads do not divide into {n_kv_heads} kv heads")
         if gate not in (False, True, None, "value", "head"):
@@ -239,6 +244,14 @@ class GatedWindowAttention(Mixer):
             raise ValueError(f"{prefix}: a learned sink and a sink of one together")
         if chunk is not None and chunk <= 0:
             raise ValueError(f"{prefix}: chunks of {chunk} positions")
+        if values_are_keys and ((v_dim or dim) != dim or shared_kv):
+            raise ValueError(f"{prefix}: values that are the keys have their size ({v_dim} and {dim}) and belong to the layer")
+        if qk_norm_whole and qk_norm_eps is None:
+            raise ValueError(f"{prefix}: a norm over all heads needs its eps")
+        if q_temp is not None and int(q_temp[1]) <= 0:
+            raise ValueError(f"{prefix}: a query temperature that steps every {q_temp[1]} positions")
+        self.qk_norm_whole, self.values_are_keys = bool(qk_norm_whole), bool(values_are_keys)
+        self.q_temp = None if q_temp is None else (float(q_temp[0]), int(q_temp[1]))
         self.prefix, self.hidden = prefix, hidden
         self.nh, self.nkv, self.dim, self.vdim = n_heads, n_kv_heads, dim, v_dim or dim
         self.position = position or NoPosition()
@@ -266,7 +279,9 @@ class GatedWindowAttention(Mixer):
 
     def _biased(self):
         """The pieces of the fused projection that carry a bias: q, and k and v where the layer has them."""
-        return [("q", self.nh * self.dim)] + ([] if self.shared_kv else [("k", self.nkv * self.dim), ("v", self.nkv * self.vdim)])
+        k = [] if self.shared_kv else [("k", self.nkv * self.dim)]
+        v = [] if self.shared_kv or self.values_are_keys else [("v", self.nkv * self.vdim)]
+        return [("q", self.nh * self.dim)] + k + v
 
     def _widths(self):
         gate = {None: 0, "head": self.nh, "value": self.nh * self.vdim}[self.gate]
@@ -281,9 +296,10 @@ class GatedWindowAttention(Mixer):
         if self.out_bias:
             specs[self._n("o", True)] = TensorSpec((self.hidden,), "bias")
         if self.qk_norm_eps is not None:
-            specs[self._n("q_norm")] = TensorSpec((self.dim,), "gain")
+            whole = self.qk_norm_whole
+            specs[self._n("q_norm")] = TensorSpec((self.nh * self.dim if whole else self.dim,), "gain")
             if not self.shared_kv:
-                specs[self._n("k_norm")] = TensorSpec((self.dim,), "gain")
+                specs[self._n("k_norm")] = TensorSpec((self.nkv * self.dim if whole else self.dim,), "gain")
         if self.sink:
             specs[self._n("sink")] = TensorSpec((self.nh,), "bias")
         specs.update(self.position.tensor_specs())
@@ -300,7 +316,7 @@ class GatedWindowAttention(Mixer):
         if self.qk_norm_eps is not None:
             self.q_gain = get(self._n("q_norm")).float().contiguous()
             # (a layer without keys of its own hands the intake its query gain twice; the key gain is never read)
-            self.k_gain = self.q_gain if self.shared_kv else get(self._n("k_norm")).float().contiguous()
+            self.k_gain = self.q_gain[:self.nkv * self.dim] if self.shared_kv else get(self._n("k_norm")).float().contiguous()
         if self.sink:
             self.sinks = get(self._n("sink")).float().contiguous()
         self.position.load(get)
@@ -336,7 +352,8 @@ class GatedWindowAttention(Mixer):
         table = ctx.page_table(cache.group)
         ops.window_intake(proj, self.b_in, q, cache.k_pages, cache.v_pages, table, ctx.tok_seq, ctx.tok_pos,
                           self.q_gain, self.k_gain, self.qk_norm_eps or 0.0, self.nh, self.nkv, self.dim, self.vdim,
-                          write_kv=owner, rotation=self.position.tables(h.device), pairs=self.position.pairing == "pairs")
+                          write_kv=owner, rotation=self.position.tables(h.device), pairs=self.position.pairing == "pairs",
+                          norm_whole=self.qk_norm_whole, values_are_keys=self.values_are_keys, q_temp=self.q_temp)
         o = torch.empty((N, self.nh * self.vdim), dtype=act, device=h.device)
         at = sum(n for _, n in self._biased())
         gate = proj[:, at:at + self._widths()[-1][1]] if self.gate else None

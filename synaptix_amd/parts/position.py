@@ -91,6 +91,16 @@ class LogDistanceBias(Position):
         return self.r1, self.r2
 
 
+class LinearDistanceBias(Position):
+    """No rotation; the score of query position i and key position j <= i gets  - slope_h (i - j)  with fixed slopes
+    slope_h = 2^(-8 (h + 1) / heads)."""
+    capturable = True
+
+    def score_slopes(self, n_heads: int, device):
+        h = torch.arange(1, n_heads + 1, dtype=torch.float64)
+        return torch.exp2(-8.0 * h / n_heads).to(device=device, dtype=torch.float32)
+
+
 class RotaryInterleaved(Position):
     """A rotation of the pairs (2i, 2i + 1), i < dims / 2, of a vector's first `dims` values by the angle
     t_i = position * base^(-2i / dims), as a complex multiplication (x_2i + j x_2i+1) e^(j t_i); what lies behind `dims`
@@ -133,7 +143,8 @@ class RotaryScaledHalfSplit(Position):
         rate_i = f_i / factor * ramp_i + f_i * (1 - ramp_i)
 
     and cos and sin both carry the factor 0.1 ln(factor) + 1.  factor None: the plain rates, no factor on cos and sin.
-    Angles are position * rate in 32-bit; tables [capacity, dims / 2], kept once for equal constants."""
+    Angles are position * rate in 32-bit; tables [capacity, dims / 2], kept once for equal constants.  (The tables do not
+    depend on which values are paired: RotaryScaledInterleaved turns pairs with them.)"""
     capturable = True
     _shared: dict = {}
 
@@ -178,6 +189,11 @@ class RotaryScaledHalfSplit(Position):
             cos, sin = self.host_tables()
             self._shared[key] = (torch.from_numpy(cos).to(device), torch.from_numpy(sin).to(device))
         return self._shared[key]
+
+
+class RotaryScaledInterleaved(RotaryScaledHalfSplit):
+    """The same stretched rotation over the pairs (2i, 2i + 1)."""
+    pairing = "pairs"
 
 
 class RotaryByWavelength(Position):

@@ -10,6 +10,10 @@ rate for every (head, key channel), made by a product through a narrow middle, a
 a step sigmoid(W_b h); each head's read-out is divided by its root mean square, times a gain, times the sigmoid of a
 gate that is also made through a narrow middle; then the output product.
 
+HeadDeltaMixer: the delta rule with one decay a head, exp(-exp(A) softplus(W_a h + bias)); each head's read-out is divided
+by its root mean square, times a gain, times silu(W_g h); everything in front of the cell is one fused projection
+[q | k | v | gate | step | decay].
+
 Step sizes, decays, gates, unit norms, states and everything between the projections and the output product are 32-bit
 in both engine types.  A sequence's state (the matrix, and the convolution's last inputs) starts at zero when its slot
 is taken and is carried from step to step.
@@ -21,8 +25,8 @@ import torch
 from ..kernels import ops
 from ..weights.source import TensorSpec
 from .base import StateNeed
-from .linear import linear, linear_for_sum
-from .mixer import Mixer, _projection
+from .linear import linear, linear_for_sum, deferred_product
+from .mixer import Mixer, _projection, _whole_fragments
 
 
 def conv_state_need(taps: int, channels: int) -> StateNeed:
@@ -189,3 +193,73 @@ class ChannelDeltaMixer(Mixer):
         o = torch.empty((N, H * self.vdim), dtype=h.dtype, device=h.device)
         ops.head_norm_gate(raw, self.gain, self.norm_eps, wide[:, H * self.dim:], o, H, self.vdim)
         return linear_for_sum(o, self.w_o)
+
+
+class HeadDeltaMixer(Mixer):
+    takes_scaled_rows = True      # (the products at both ends take a norm's halves: parts.linear)
+    capturable = True
+
+    NAMES = {"q": "q", "k": "k", "v": "v", "conv": ".conv", "g": "g", "b": "b", "a": "a", "a_bias": "dt_bias",
+             "a_log": "A_log", "norm": "norm", "o": "o"}
+    UNIT_EPS = 1e-6       # inside the root of the unit norm of q and k
+
+    def __init__(self, prefix: str, hidden: int, n_heads: int, n_key_heads: int, dim: int, vdim: int, taps: int, *,
+                 norm_eps: float, q_scale: float | None = None, names: dict | None = None):
+        if n_key_heads <= 0 or n_heads % n_key_heads:
+            raise ValueError(f"{prefix}: {n_heads} heads do not divide into {n_key_heads} key heads")
+        self.prefix, self.hidden = prefix, hidden
+        self.nh, self.nk, self.dim, self.vdim, self.taps = n_heads, n_key_heads, dim, vdim, taps
+        self.norm_eps = float(norm_eps)
+        self.q_scale = float(q_scale) if q_scale is not None else dim ** -0.5
+        self.channels = 2 * n_key_heads * dim + n_heads * vdim
+        self.names = dict(self.NAMES, **(names or {}))
+        self.w_in = self.w_o = self.conv = self.a_bias = self.a_log = self.gain = None
+
+    def _n(self, key):
+        return self.prefix + self.names[key]
+
+    def _qkv(self):
+        return [("q", self.nk * self.dim), ("k", self.nk * self.dim), ("v", self.nh * self.vdim)]
+
+    def _rows(self):
+        """The fused projection's pieces, in their order."""
+        return self._qkv() + [("g", self.nh * self.vdim), ("b", self.nh), ("a", self.nh)]
+
+    def tensor_specs(self):
+        specs = {self._n(k): TensorSpec((n, self.hidden)) for k, n in self._rows()}
+        specs.update({self._n(k) + self.names["conv"]: TensorSpec((n, self.taps), "filter") for k, n in self._qkv()})
+        specs.update({self._n("a_bias"): TensorSpec((self.nh,), "bias"), self._n("a_log"): TensorSpec((self.nh,), "rate"),
+                      self._n("norm"): TensorSpec((self.vdim,), "gain"),
+                      self._n("o"): TensorSpec((self.hidden, self.nh * self.vdim))})
+        return specs
+
+    def load(self, get):
+        self.w_in = _projection(_whole_fragments(torch.cat([get(self._n(k)) for k, _ in self._rows()], 0)))
+        self.w_o = _projection(get(self._n("o")))
+        self.conv = torch.cat([get(self._n(k) + self.names["conv"]) for k, _ in self._qkv()], 0).float().contiguous()
+        self.a_bias = get(self._n("a_bias")).float().contiguous()
+        self.a_log = get(self._n("a_log")).float().contiguous()
+        self.gain = get(self._n("norm")).float().repeat(self.nh).contiguous()        # one gain for all heads
+
+    def cache_need(self):
+        return (conv_state_need(self.taps, self.channels), StateNeed((self.nh, self.dim, self.vdim)))
+
+    def check(self, dtype):
+        if self.dim > ops.SCAN_MAX_ROWS or not 1 <= self.taps <= ops.SHORT_CONV_MAX_TAPS:
+            raise ValueError(f"{self.prefix}: keys of {self.dim} values (at most {ops.SCAN_MAX_ROWS}), {self.taps} taps "
+                             f"(at most {ops.SHORT_CONV_MAX_TAPS})")
+
+    def forward(self, h, ctx, cache, owner=True):
+        N, H, C, E = h.shape[0], self.nh, self.channels, self.nh * self.vdim
+        conv_state, cell = cache
+        proj = linear(h, self.w_in, torch.float32)          # [N, q | k | v | gate | step | decay] float
+        qkv = torch.empty((N, C), dtype=torch.float32, device=proj.device)
+        ops.short_conv(proj[:, :C], self.conv, None, conv_state.state, ctx.tok_seq, ctx.tok_pos, ctx.seq_start,
+                       ctx.seq_past, ctx.seq_slot, qkv, silu=True)
+        raw = torch.empty((N, E), dtype=torch.float32, device=proj.device)
+        ops.head_delta_scan(qkv, proj[:, C + E:], proj[:, C + E + H:], self.a_bias, self.a_log, self.q_scale, self.UNIT_EPS,
+                            cell.state, ctx.seq_start, ctx.seq_slot, raw, H, self.nk, self.dim, self.vdim,
+                            single_tokens=ctx.one_token_each)
+        o = torch.empty((N, E), dtype=h.dtype, device=proj.device)
+        ops.head_norm_gate(raw, self.gain, self.norm_eps, proj[:, C:], o, H, self.vdim, silu=True)
+        return deferred_product(o, self.w_o)

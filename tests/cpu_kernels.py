@@ -58,7 +58,8 @@ def swiglu(gate_up, out, activation="silu"):
     out.copy_((g / (1 + torch.exp(-g)) * u).to(out.dtype))
 
 
-def gemm(x, w, out, force_simt=False):
+def gemm(x, w, out, force_simt=False, point=None):
+    assert point is None
     w = _rows(w)
     if out.dim() == 3:                      # partial sums over slices of K
         S, K = out.shape[0], x.shape[1]
@@ -82,7 +83,8 @@ def gemm_swiglu(x, w_paired, out, activation="silu"):
     out.copy_((g / (1 + torch.exp(-g)) * u).to(out.dtype))
 
 
-def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, resid_norm=None):
+def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, resid_norm=None, point=None):
+    assert point is None
     from synaptix_amd.kernels import ops
     w = ops.unpack_weight(wp)
     factor = None
