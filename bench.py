@@ -2,7 +2,7 @@
 """Throughput of the engine at a Qwen3 shape with random bf16 weights on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--shape 8b|4b|32b] [--batch 8] [--layers L]
-    python bench.py --design bizipel|kamivik|repolix|nilepel [--sizes small,mid,large] [--prompt 2048] [--batch 8] [--window 1024]
+    python bench.py --design bizipel|kamivik|repolix|nilepel|pizunex [--sizes small,mid,large] [--prompt 2048] [--batch 8] [--window 1024]
 
 --shape 8b (the default) and 32b: a step is one decode step of `batch` sequences, each after a
 2,048-token prompt of uniform ids, run through the same captured graph and host loop that
@@ -37,6 +37,10 @@ head turned with stretched long waves, a sink, a gate a head), latent attention 
 window), attention over runs of `window` positions (pairs turned, a sink), windowed attention again on the first layer's
 keys and values; the first and third layers with a bounded dense feed-forward, the others with silu experts of which each
 token uses top - 1 within one of two groups beside a gated shared expert (together the dense feed-forward's width).
+--design pizunex: the same for the Pizunex design: layers in the order delta rule with one decay a head (the heads, kv heads and
+head size of the attention), attention whose values are its keys (norms over whole projections, a query temperature, a soft
+cap, a linear distance bias, the window), latent attention (a latent of 512 beside 64 turned values, a query latent of 3/8
+of the width), delta rule; every layer with an ungated feed-forward (squared relu) of the dense feed-forward's width.
 
 Method after the reference's own harnesses (crates/synaptix-models/llm/qwen3/examples/format_perf.rs:41-122,
 crates/synaptix-cli/src/commands/bench.rs:35-96): synthetic ids, warm-up first, device synchronised
@@ -188,6 +192,7 @@ SIDE_BY_SIDE_SIZES = {     # layers, width, heads, kv heads, head size, feed-for
 
 KAMIVIK_EXPERTS = {"small": (4, 1024), "mid": (4, 2048), "large": (6, 2048)}      # (top, an expert's width); 8 x top experts
 REPOLIX_ORDER = ("mamba2", "channel_delta", "attention", "mamba2")
+PIZUNEX_ORDER = ("delta", "attention", "latent_attention", "delta")
 NILEPEL_ORDER = ("attention_2", "latent_attention", "attention", "attention_2")
 
 
@@ -205,7 +210,7 @@ def design_configs(design, size, window, context):
     layers have latent attention (a latent of 512, 64 rotated values, unrotated keys and values of the head size; every
     second layer with the window) and a mixture of experts whose active width equals the dense feed-forward's."""
     from synaptix_amd import Qwen3Config
-    from synaptix_amd.config import BizipelConfig, KamivikConfig, RepolixConfig, NilepelConfig
+    from synaptix_amd.config import BizipelConfig, KamivikConfig, RepolixConfig, NilepelConfig, PizunexConfig
     L, W, nh, nkv, hd, ff, V = SIDE_BY_SIDE_SIZES[size]
     qwen = Qwen3Config.from_dict(dict(_COMMON, num_hidden_layers=L, hidden_size=W, num_attention_heads=nh,
                                       num_key_value_heads=nkv, head_dim=hd, intermediate_size=ff, vocab_size=V,
@@ -243,6 +248,18 @@ def design_configs(design, size, window, context):
         nil = NilepelConfig.from_dict({"architecture": "Nilepel", "vocab": V, "width": W, "norm": {"eps": 1e-6},
                                        "embedding": {"scale": float(W) ** 0.5}, "layers": layers})
         return qwen, nil
+    if design == "pizunex":
+        mixers = {"delta": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "conv": 4},
+                  "attention": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "softcap": 50.0,
+                                "mask": {"size": window}, "q_temp": {"coef": 0.1, "every": 1024}},
+                  "latent_attention": {"heads": nh, "dim": hd, "rot_dim": 64, "vdim": hd, "kv_rank": 512, "q_rank": 3 * W // 8,
+                                       "scale": (hd + 64) ** -0.5,
+                                       "rot": {"base": 10000.0, "dims": 64,
+                                               "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+        layers = [{"type": PIZUNEX_ORDER[i % 4], "mixer": mixers[PIZUNEX_ORDER[i % 4]], "mlp": {"kind": "dense", "ff": ff}}
+                  for i in range(L)]
+        piz = PizunexConfig.from_dict({"architecture": "Pizunex", "vocab": V, "width": W, "norm": {"eps": 1e-6}, "layers": layers})
+        return qwen, piz
     if design == "kamivik":
         top, eff = KAMIVIK_EXPERTS[size]
         layers = []
@@ -375,7 +392,7 @@ def main() -> int:
                     help="the longest sequence (positions and cache a sequence; the contract's run has 8,192)")
     ap.add_argument("--no-points", action="store_true", help="skip decode at batch 1 and 64")
     ap.add_argument("--no-graph", action="store_true", help="launch every kernel of a decode step from the host")
-    ap.add_argument("--design", default=None, choices=["bizipel", "kamivik", "repolix", "nilepel"],
+    ap.add_argument("--design", default=None, choices=["bizipel", "kamivik", "repolix", "nilepel", "pizunex"],
                     help="another run than the default one: this design beside the Qwen3 decoder at equal layer sizes")
     ap.add_argument("--sizes", default="small,mid,large", help="with --design: which of small, mid, large")
     ap.add_argument("--window", type=int, default=1024, help="with --design: the keys a query of the new design sees")

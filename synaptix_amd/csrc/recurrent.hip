@@ -6,7 +6,7 @@
 //   state_space_scan   a scalar decay a head:   S <- exp(-exp(A) dt) S + dt B x^T,  y = S^T C + D x      (S: N x P)
 //   channel_delta_scan a decay for every key channel and the delta rule:
 //                      S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q                 (S: D x P)
-//   head_delta_scan    the same with one decay a head, S <- g S
+//   head_delta_scan    the same with one decay a head, S <- g S (prompts in chunks on the matrix cores)
 //   diff_heads         two softmax maps over the same values, o = rms_norm(a1 - lambda a2) (1 - c)
 //
 // Everything here is 32-bit FMA: inputs are the float sums of the projections, states are float.  The scans walk a
@@ -478,6 +478,300 @@ delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict__ beta,
   }
 }
 
+// ---------------------------------------------------------------- delta rule with one decay a head, prompts in chunks
+// With a decay for the whole state a chunk of C tokens is a few small products.  From the state S before the chunk, with
+// G_t = g_1 .. g_t and G_tj = g_(j+1) .. g_t (products of at most C decays, no quotient):
+//   u_t = b_t (v_t - G_t S^T k_t - sum_(j<t) G_tj (k_t . k_j) u_j)        so  (I + L) U = diag(b) (V - diag(G) K S)
+//   o_t = G_t S^T q_t + sum_(j<=t) G_tj (q_t . k_j) u_j                      with L_tj = b_t G_tj (k_t . k_j), j < t
+//   S'  = G_C S + sum_j G_Cj k_j u_j^T
+// (the unrolled recurrence; the triangular system of the delta rule's chunked form: S. Yang, B. Wang, Y. Zhang, Y. Shen,
+// Y. Kim, "Parallelizing Linear Transformers with the Delta Rule over Sequence Length").  T = (I + L)^-1 diag(b),
+// A_tj = G_tj (q_t . k_j) and the decays do not depend on the state: head_delta_chunks_kernel makes them for all chunks side by
+// side.  head_delta_carry_kernel then walks the chunks:  U = T (V - diag(G) K S),  O = diag(G) Q S + A U,
+// S <- G_C S + K^T diag(G_Cj) U, on the matrix cores in 32-bit (16x16x4).
+//
+// C = 16 is that instruction's side.  Everything lies in the order of its operands: a wave holds 16 columns of a head's
+// state as accumulators (lane = 16 g + n has rows 16 i + 4 g + j of column n), and an accumulator is also the B operand of the
+// next product if the k index of step j counts the rows 4 g + j, so neither the state nor U ever moves between lanes.  The
+// A operands of four steps are then four consecutive values of a row: "fragments" [tile][lane][4] of 1 KB.
+#define HDC 16
+typedef f32x4 hd_frag;
+
+// floats of one (chunk, key head): K, Q and K^T in fragments; of one (chunk, head): T, A, [G_t], [G_Cj]
+__host__ __device__ __forceinline__ size_t hd_key_floats(int NT) { return (size_t)3 * NT * 256; }
+#define HD_HEAD_FLOATS (2 * 256 + 2 * HDC)
+
+// Which sequence and chunk a place of the chunk arrays is: sequence b's chunks begin at seq_start[b] / C + b, which leaves
+// room for every sequence's last, partly filled chunk.  False for places of no chunk.
+__device__ __forceinline__ bool hd_chunk_of(int place, const int* __restrict__ seq_start, int n_seqs, int& first, int& n) {
+  for (int b = 0; b < n_seqs; ++b) {
+    const int s0 = seq_start[b], s1 = seq_start[b + 1], at = place - (s0 / HDC + b);
+    if (at >= 0 && at * HDC < s1 - s0) {
+      first = s0 + at * HDC, n = min(HDC, s1 - first);
+      return true;
+    }
+  }
+  return false;
+}
+
+// One workgroup a (chunk, key head), and the heads that read it.
+__global__ void __launch_bounds__(256)
+head_delta_chunks_kernel(const float* __restrict__ qkv, const float* __restrict__ beta, int beta_stride,
+                         const float* __restrict__ a, int a_stride, const float* __restrict__ a_bias,
+                         const float* __restrict__ a_log, float q_scale, float unit_eps, const int* __restrict__ seq_start,
+                         int n_seqs, float* __restrict__ keys, float* __restrict__ heads, int H, int K, int D, int E, int NT) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int LDD = 16 * NT + 1;
+  float* ks = lds;                        // [C][LDD] unit keys, zeros beyond the keys and the chunk's tokens
+  float* qs = ks + HDC * LDD;             // [C][LDD] unit queries times q_scale
+  float* kk = qs + HDC * LDD;             // [C][C + 1] k_t . k_j
+  float* qk = kk + HDC * (HDC + 1);       // [C][C + 1] q_t . k_j
+  float* Ls = qk + HDC * (HDC + 1);       // [4 waves][C][C + 1]
+  float* gs = Ls + 4 * HDC * (HDC + 1);   // [4 waves][2][C] decays, steps
+  int first, n;
+  if (!hd_chunk_of(blockIdx.x, seq_start, n_seqs, first, n)) return;      // (the whole workgroup)
+  const int kvh = blockIdx.y, tid = threadIdx.x, wave = tid / SYN_WAVE, lane = tid % SYN_WAVE;
+  const int width = 2 * K * D + H * E;
+  for (int t = wave; t < HDC; t += 4) {
+    const float* qr = qkv + (size_t)(first + min(t, n - 1)) * width + kvh * D;
+    const float* kr = qr + K * D;
+    float q[RC_ROWS_MAX / SYN_WAVE], k[RC_ROWS_MAX / SYN_WAVE], sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < RC_ROWS_MAX / SYN_WAVE; ++i) {
+      const int d = lane + i * SYN_WAVE;
+      const bool in = t < n && d < D;
+      q[i] = in ? qr[d] : 0.f, k[i] = in ? kr[d] : 0.f;
+      sq = fmaf(q[i], q[i], sq), sk = fmaf(k[i], k[i], sk);
+    }
+    sq = wave_sum(sq), sk = wave_sum(sk);
+    const float iq = q_scale / sqrtf(sq + unit_eps), ik = 1.f / sqrtf(sk + unit_eps);
+#pragma unroll
+    for (int i = 0; i < RC_ROWS_MAX / SYN_WAVE; ++i) {
+      const int d = lane + i * SYN_WAVE;
+      if (d < 16 * NT) qs[t * LDD + d] = q[i] * iq, ks[t * LDD + d] = k[i] * ik;
+    }
+  }
+  __syncthreads();
+  // the fragments of K (row m = token, k = 4 g + j), Q and K^T (row m = key value, k = token 4 g + j)
+  float* kf = keys + ((size_t)blockIdx.x * K + kvh) * hd_key_floats(NT);
+  for (int e = tid; e < NT * 64; e += 256) {
+    const int tile = e / 64, m = e % 16, g = (e % 64) / 16;
+    hd_frag fk, fq, ft;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      fk[j] = ks[m * LDD + 16 * tile + 4 * g + j];
+      fq[j] = qs[m * LDD + 16 * tile + 4 * g + j];
+      ft[j] = ks[(4 * g + j) * LDD + 16 * tile + m];
+    }
+    ((hd_frag*)kf)[e] = fk, ((hd_frag*)kf)[NT * 64 + e] = fq, ((hd_frag*)kf)[2 * NT * 64 + e] = ft;
+  }
+  {
+    const int t = tid / HDC, j = tid % HDC;
+    float dk = 0.f, dq = 0.f;
+    for (int d = 0; d < D; ++d) {
+      const float kj = ks[j * LDD + d];
+      dk = fmaf(ks[t * LDD + d], kj, dk), dq = fmaf(qs[t * LDD + d], kj, dq);
+    }
+    kk[t * (HDC + 1) + j] = dk, qk[t * (HDC + 1) + j] = dq;
+  }
+  __syncthreads();
+  // a wave a head; what its lanes exchange through LDS is the wave's own (every wave takes the same number of turns, so
+  // the barriers are the workgroup's)
+  const int rep = H / K;
+  float* L = Ls + wave * HDC * (HDC + 1);
+  float* gd = gs + wave * 2 * HDC;
+  for (int r0 = 0; r0 < rep; r0 += 4) {
+    const bool on = r0 + wave < rep;
+    const int head = kvh * rep + min(r0 + wave, rep - 1);
+    if (lane < HDC) {       // tokens beyond the chunk's: nothing decays, nothing is written
+      const size_t tok = first + min(lane, n - 1);
+      gd[lane] = lane < n ? expf(-expf(a_log[head]) * rc_softplus(a[tok * a_stride + head] + a_bias[head])) : 1.f;
+      gd[HDC + lane] = lane < n ? 1.f / (1.f + expf(-beta[tok * beta_stride + head])) : 0.f;
+    }
+    __syncthreads();
+    float* hf = heads + ((size_t)blockIdx.x * H + head) * HD_HEAD_FLOATS;
+    const int j = lane % HDC;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = 4 * (lane / HDC) + i;
+      float dec = t >= j ? 1.f : 0.f;
+      for (int x = j + 1; x <= t; ++x) dec *= gd[x];
+      L[t * (HDC + 1) + j] = t > j ? gd[HDC + t] * dec * kk[t * (HDC + 1) + j] : 0.f;
+      if (on) {
+        hf[256 + ((j / 4) * 16 + t) * 4 + j % 4] = dec * qk[t * (HDC + 1) + j];       // A, row t, k = j
+        if (t == HDC - 1) hf[2 * 256 + HDC + j] = dec;                                 // G_Cj
+        if (j == 0) hf[2 * 256 + t] = dec * gd[0];                                     // G_t
+      }
+    }
+    __syncthreads();
+    if (lane < HDC) {       // column j of (I + L)^-1, row after row
+      float col[HDC];
+#pragma unroll
+      for (int t = 0; t < HDC; ++t) {
+        float v = t == j ? 1.f : 0.f;
+#pragma unroll
+        for (int x = 0; x < t; ++x) v = fmaf(-L[t * (HDC + 1) + x], col[x], v);
+        col[t] = v;
+      }
+      const float step = gd[HDC + j];
+      if (on) {
+#pragma unroll
+        for (int t = 0; t < HDC; ++t) hf[((j / 4) * 16 + t) * 4 + j % 4] = col[t] * step;      // T, row t, k = j
+      }
+    }
+    __syncthreads();
+  }
+}
+
+__device__ __forceinline__ f32x4 hd_mfma(float a, float b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+// One chunk's operands in a wave's registers.
+template <int TPW, int CG>
+struct HdOperands {
+  hd_frag k[TPW], q[TPW], kt[TPW], T, A;
+  f32x4 gt, gc, v[CG];  // G_t and G_Cj of the tokens 4 g + j, their values in this lane's columns
+};
+
+// A workgroup for CG groups of 16 columns of a (sequence, head): two where there are enough workgroups even so, since they
+// share the keys' operands.  W waves hold TPW tiles of 16 rows of the state each: what a wave's
+// rows give to K S and Q S is summed through LDS (two buffers in turns: one barrier a chunk), then every wave makes U and
+// updates its rows; one more wave makes and stores the outputs meanwhile.  The operands are asked for two chunks ahead.
+template <int TPW, int W, int CG>
+__global__ void __launch_bounds__((W + 1) * SYN_WAVE)
+head_delta_carry_kernel(const float* __restrict__ qkv, const float* __restrict__ keys, const float* __restrict__ heads,
+                        float* __restrict__ state, int state_rows, const int* __restrict__ seq_start,
+                        const int* __restrict__ seq_slot, float* __restrict__ o, int H, int K, int D, int E) {
+  constexpr int NT = TPW * W;
+  __shared__ __attribute__((aligned(16))) f32x4 part[2][W][2][CG][SYN_WAVE];
+  const int head = blockIdx.x, b = blockIdx.z, wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE;
+  const bool holds = wave < W;                       // (else the wave of the outputs)
+  const int g = lane / 16, col = blockIdx.y * 16 * CG + lane % 16;       // (this lane's columns: col, col + 16)
+  const int s0 = seq_start[b], n_new = seq_start[b + 1] - s0;
+  if (n_new <= 0) return;                            // (the whole workgroup)
+  int slot = seq_slot[b];
+  if (slot < 0 || slot >= state_rows) slot = state_rows - 1;
+  const int kvh = head / (H / K), width = 2 * K * D + H * E;
+  float* Sg = state + ((size_t)slot * H + head) * D * E;
+  f32x4 S[CG][TPW];
+#pragma unroll
+  for (int y = 0; y < CG; ++y)
+#pragma unroll
+    for (int i = 0; i < TPW; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = 16 * (wave * TPW + i) + 4 * g + j, c = col + 16 * y;
+        S[y][i][j] = (holds && c < E && d < D) ? Sg[(size_t)d * E + c] : 0.f;
+      }
+  const int chunk0 = s0 / HDC + b, n_chunks = (n_new + HDC - 1) / HDC;
+  const float* vp = qkv + (size_t)s0 * width + 2 * K * D + head * E;
+  float* op = o + (size_t)s0 * H * E + head * E + col;
+  auto ask = [&](HdOperands<TPW, CG>& x, int c) {
+    c = min(c, n_chunks - 1);
+    const float* hf = heads + ((size_t)(chunk0 + c) * H + head) * HD_HEAD_FLOATS;
+    if (holds) {
+      const hd_frag* kf = (const hd_frag*)(keys + ((size_t)(chunk0 + c) * K + kvh) * hd_key_floats(NT)) + wave * TPW * 64 + lane;
+#pragma unroll
+      for (int i = 0; i < TPW; ++i) x.k[i] = kf[i * 64], x.q[i] = kf[(NT + i) * 64], x.kt[i] = kf[(2 * NT + i) * 64];
+      x.gc = ((const f32x4*)(hf + 2 * 256 + HDC))[g];
+    } else {
+      x.A = ((const hd_frag*)(hf + 256))[lane];
+    }
+    x.T = ((const hd_frag*)hf)[lane];
+    x.gt = ((const f32x4*)(hf + 2 * 256))[g];
+#pragma unroll
+    for (int y = 0; y < CG; ++y)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)      // (T has zeros for tokens beyond the last; columns beyond are not stored)
+        x.v[y][j] = vp[(size_t)min(c * HDC + 4 * g + j, n_new - 1) * width + min(col + 16 * y, E - 1)];
+  };
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  auto step = [&](const HdOperands<TPW, CG>& x, int c, int at) {
+    if (holds) {
+#pragma unroll
+      for (int y = 0; y < CG; ++y) {
+        f32x4 ks[2] = {zero, zero}, qs[2] = {zero, zero};
+#pragma unroll
+        for (int i = 0; i < TPW; ++i)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            ks[j & 1] = hd_mfma(x.k[i][j], S[y][i][j], ks[j & 1]);
+            qs[j & 1] = hd_mfma(x.q[i][j], S[y][i][j], qs[j & 1]);
+          }
+        part[at][wave][0][y][lane] = ks[0] + ks[1];
+        part[at][wave][1][y][lane] = qs[0] + qs[1];
+      }
+    }
+    __syncthreads();
+    f32x4 u[CG];
+#pragma unroll
+    for (int y = 0; y < CG; ++y) {
+      f32x4 sum = part[at][0][0][y][lane];
+#pragma unroll
+      for (int w = 1; w < W; ++w) sum += part[at][w][0][y][lane];
+      const f32x4 r = x.v[y] - x.gt * sum;
+      u[y] = zero;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) u[y] = hd_mfma(x.T[j], r[j], u[y]);
+    }
+    if (holds) {
+      const float whole = __shfl(x.gt[3], 48, SYN_WAVE);        // G_C: the last token's
+#pragma unroll
+      for (int y = 0; y < CG; ++y) {
+        const f32x4 uc = x.gc * u[y];
+#pragma unroll
+        for (int i = 0; i < TPW; ++i) S[y][i] *= whole;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int i = 0; i < TPW; ++i) S[y][i] = hd_mfma(x.kt[i][j], uc[j], S[y][i]);
+      }
+    } else {
+#pragma unroll
+      for (int y = 0; y < CG; ++y) {
+        f32x4 out = part[at][0][1][y][lane];
+#pragma unroll
+        for (int w = 1; w < W; ++w) out += part[at][w][1][y][lane];
+        out *= x.gt;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) out = hd_mfma(x.A[j], u[y][j], out);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int t = c * HDC + 4 * g + j;
+          if (t < n_new && col + 16 * y < E) op[(size_t)t * H * E + 16 * y] = out[j];
+        }
+      }
+    }
+  };
+  HdOperands<TPW, CG> even, odd;
+  ask(even, 0), ask(odd, 1);
+  for (int c = 0; c < n_chunks; c += 2) {
+    step(even, c, 0);
+    ask(even, c + 2);
+    if (c + 1 < n_chunks) {
+      step(odd, c + 1, 1);
+      ask(odd, c + 3);
+    }
+  }
+#pragma unroll
+  for (int y = 0; y < CG; ++y)
+#pragma unroll
+    for (int i = 0; i < TPW; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = 16 * (wave * TPW + i) + 4 * g + j, c = col + 16 * y;
+        if (holds && c < E && d < D) Sg[(size_t)d * E + c] = S[y][i][j];
+      }
+}
+
+static int hd_tiles(int D) {      // tiles of 16 key values: what the walk is built for
+  const int need = (D + 15) / 16;
+  for (int nt : {1, 2, 4, 8, 12, 16})
+    if (need <= nt) return nt;
+  return 0;
+}
+
 template <bool CHANNEL>
 static int delta_scan(const char* name, const float* qkv, const float* beta, int beta_stride, const float* a, int a_stride,
                       const float* a_bias, const float* a_log, float q_scale, float unit_eps, float* state, int state_rows,
@@ -524,12 +818,52 @@ SYN_EXPORT int syn_channel_delta_scan(const float* qkv, const float* beta, int b
                           state_rows, seq_start, seq_slot, n_seqs, longest, o, H, K, D, E, stream);
 }
 
+// floats of scratch memory of a call over prompts
+SYN_EXPORT long syn_head_delta_scratch(int n_tokens, int n_seqs, int H, int K, int D) {
+  return ((long)n_tokens / HDC + n_seqs) * (K * (long)hd_key_floats(hd_tiles(D)) + H * (long)HD_HEAD_FLOATS);
+}
+
+// scratch == nullptr: token by token in one launch (single tokens); else in chunks
 SYN_EXPORT int syn_head_delta_scan(const float* qkv, const float* beta, int beta_stride, const float* a, int a_stride,
                                    const float* a_bias, const float* a_log, float q_scale, float unit_eps, float* state,
                                    int state_rows, const int* seq_start, const int* seq_slot, int n_seqs, int longest,
-                                   float* o, int H, int K, int D, int E, hipStream_t stream) {
-  return delta_scan<false>("head_delta_scan", qkv, beta, beta_stride, a, a_stride, a_bias, a_log, q_scale, unit_eps, state,
-                           state_rows, seq_start, seq_slot, n_seqs, longest, o, H, K, D, E, stream);
+                                   float* o, int H, int K, int D, int E, int n_tokens, float* scratch, hipStream_t stream) {
+  if (scratch == nullptr)
+    return delta_scan<false>("head_delta_scan", qkv, beta, beta_stride, a, a_stride, a_bias, a_log, q_scale, unit_eps, state,
+                             state_rows, seq_start, seq_slot, n_seqs, longest, o, H, K, D, E, stream);
+  SYN_CHECK(n_seqs > 0 && n_tokens > 0 && H > 0 && K > 0 && D > 0 && E > 0, "head_delta_scan: empty input");
+  SYN_CHECK(H % K == 0, "head_delta_scan: %d heads do not divide into %d key heads", H, K);
+  SYN_CHECK(D <= RC_ROWS_MAX, "head_delta_scan: keys of %d values (at most %d)", D, RC_ROWS_MAX);
+  SYN_CHECK(beta_stride >= H && a_stride >= H && state_rows > 0, "head_delta_scan: rows of %d and %d values for %d heads",
+            beta_stride, a_stride, H);
+  SYN_CHECK((uintptr_t)scratch % 16 == 0, "head_delta_scan: the scratch memory is not aligned");
+  const int NT = hd_tiles(D), chunks = n_tokens / HDC + n_seqs;
+  float* keys = scratch;
+  float* heads = scratch + (size_t)chunks * K * hd_key_floats(NT);
+  const size_t bytes = (2 * HDC * (16 * NT + 1) + 6 * HDC * (HDC + 1) + 8 * HDC) * sizeof(float);
+  head_delta_chunks_kernel<<<dim3(chunks, K), 256, bytes, stream>>>(qkv, beta, beta_stride, a, a_stride, a_bias, a_log, q_scale,
+                                                                    unit_eps, seq_start, n_seqs, keys, heads, H, K, D, E, NT);
+  SYN_LAUNCH_CHECK("head_delta_chunks");
+  // (a sequence's workgroups follow one another, a head's on one XCD where H is a multiple of 8: they read the same fragments)
+  const int groups = (E + 15) / 16;
+  const bool wide = (long)H * n_seqs * ((groups + 1) / 2) >= 2L * syn_compute_units();
+  const dim3 grid(H, wide ? (groups + 1) / 2 : groups, n_seqs);
+#define SYN_HD2(T, W, CG)                                                                                                    \
+  head_delta_carry_kernel<T, W, CG><<<grid, (W + 1) * SYN_WAVE, 0, stream>>>(qkv, keys, heads, state, state_rows, seq_start, \
+                                                                            seq_slot, o, H, K, D, E)
+#define SYN_HD(T, W)                      \
+  case T * W:                             \
+    if (wide) SYN_HD2(T, W, 2);           \
+    else SYN_HD2(T, W, 1);                \
+    break
+  switch (NT) {
+    SYN_HD(1, 1); SYN_HD(1, 2); SYN_HD(1, 4); SYN_HD(2, 4); SYN_HD(3, 4); SYN_HD(4, 4);
+    default: SYN_CHECK(false, "head_delta_scan: keys of %d values", D);
+  }
+#undef SYN_HD2
+#undef SYN_HD
+  SYN_LAUNCH_CHECK("head_delta_carry");
+  return 0;
 }
 
 // ---------------------------------------------------------------- two softmax maps over the same values

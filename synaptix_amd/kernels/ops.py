@@ -1144,7 +1144,8 @@ def state_space_scan(xbc, dt, dt_bias, a_log, d_skip, state, seq_start, seq_slot
 
 
 def _delta_scan(name, qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads, n_key_heads,
-                dim, vdim, n_decays, single_tokens):
+                dim, vdim, n_decays, single_tokens, tail=()):
+    """The checks and the call of both delta rules; tail: what the entry point takes behind the sizes."""
     H, K = n_heads, n_key_heads
     if K <= 0 or H % K:
         raise KernelError(f"{name}: {H} heads do not divide into {K} key heads")
@@ -1161,7 +1162,7 @@ def _delta_scan(name, qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq
     _need(out, name + ".out", _F32, (N, H * vdim))
     _call(load_library("core"), "syn_" + name, _ptr(qkv), _ptr(beta), stride, _ptr(a), a_stride, _ptr(a_bias),
           _ptr(a_log), ctypes.c_float(q_scale), ctypes.c_float(unit_eps), _ptr(state), state.shape[0], _ptr(seq_start),
-          _ptr(seq_slot), B, 1 if single_tokens else max(N, 2), _ptr(out), H, K, dim, vdim, _stream())
+          _ptr(seq_slot), B, 1 if single_tokens else max(N, 2), _ptr(out), H, K, dim, vdim, *tail, _stream())
 
 
 def channel_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads,
@@ -1179,10 +1180,22 @@ def channel_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, se
 
 
 def head_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads, n_key_heads,
-                    dim, vdim, single_tokens=False):
-    """channel_delta_scan with one decay a head: a a float view [N, >= H], a_bias float [H], S <- g S."""
+                    dim, vdim, chunked=False, scratch=None):
+    """channel_delta_scan with one decay a head: a a float view [N, >= H], a_bias float [H], S <- g S.
+    chunked: 16 tokens at a time on the matrix cores (prompts) instead of token by token (single tokens); the same sums in
+    another order, in 32-bit both.  scratch: with chunked, a function (name, floats) -> float tensor for the chunks'
+    operands (StepContext.scratch; default: a new tensor)."""
+    work = None
+    if chunked:
+        lib = load_library("core")
+        lib.syn_head_delta_scratch.restype = ctypes.c_long
+        need = lib.syn_head_delta_scratch(qkv.shape[0], seq_slot.shape[0], n_heads, n_key_heads, dim)
+        work = scratch("head_delta_chunks", need) if scratch is not None else torch.empty(need, dtype=_F32, device=qkv.device)
+        _need(work, "head_delta_scan.scratch", _F32)
+        if work.numel() < need:
+            raise KernelError(f"head_delta_scan: scratch of {work.numel()} floats, {need} are needed")
     _delta_scan("head_delta_scan", qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_start, seq_slot, out, n_heads,
-                n_key_heads, dim, vdim, n_heads, single_tokens)
+                n_key_heads, dim, vdim, n_heads, not chunked, (qkv.shape[0], _ptr(work)))
 
 
 def diff_heads(a, out, lam, eps, post, n_kv_heads, heads_per_kv, vdim):

@@ -259,7 +259,7 @@ class HeadDeltaMixer(Mixer):
         raw = torch.empty((N, E), dtype=torch.float32, device=proj.device)
         ops.head_delta_scan(qkv, proj[:, C + E:], proj[:, C + E + H:], self.a_bias, self.a_log, self.q_scale, self.UNIT_EPS,
                             cell.state, ctx.seq_start, ctx.seq_slot, raw, H, self.nk, self.dim, self.vdim,
-                            single_tokens=ctx.one_token_each)
+                            chunked=not ctx.one_token_each, scratch=ctx.scratch)
         o = torch.empty((N, E), dtype=h.dtype, device=proj.device)
         ops.head_norm_gate(raw, self.gain, self.norm_eps, proj[:, C:], o, H, self.vdim, silu=True)
         return deferred_product(o, self.w_o)

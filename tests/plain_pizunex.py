@@ -154,13 +154,16 @@ def rotate_pairs(x, f, mult=1.0, first=0):
 
 
 def latent_attention(h, w, p, c, eps):
-    """Queries through a normed latent of their own; per-head keys and values from one normed latent a token, and one
+    """Queries through a normed latent of their own (or straight from h: no q_rank); per-head keys and values from one normed latent a token, and one
     turned key part for all heads."""
     T = h.shape[0]
     H, D, R, E, C = c["heads"], c["dim"], c["rot_dim"], c["vdim"], c["kv_rank"]
     f, mult = rates(c["rot"]["base"], c["rot"]["dims"], c["rot"].get("scaling"))
-    cq = rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps)
-    q = (cq @ w[p + "uq"].T).view(T, H, D + R)
+    if c.get("q_rank") is not None:
+        q = rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps) @ w[p + "uq"].T
+    else:
+        q = h @ w[p + "q"].T
+    q = q.view(T, H, D + R)
     q = torch.cat([q[..., :D], rotate_pairs(q[..., D:], f, mult)], -1)
     down = h @ w[p + "dkv"].T
     lat = rms_norm(down[:, :C], w[p + "dkv.norm"], eps)
