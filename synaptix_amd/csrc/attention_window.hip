@@ -147,26 +147,40 @@ __global__ void window_intake_kernel(IntakeArgs a, T* __restrict__ q_out, T* __r
   intake_store<T>(a, t, tok, item, lane, gain, inv, q_out, k_pages, v_pages);
 }
 
-// norms over all query heads at once and over all key heads at once (gains [nh * dim] and [nkv * dim]): a workgroup a
-// token, which sums both squares first and then stores item after item
+// norms over all query heads at once and over all key heads at once (gains [nh * dim] and [nkv * dim]): a workgroup sums
+// both squares of its token's row first and then stores its share of the items (blockIdx.y of gridDim.y: single tokens
+// have several workgroups a token, which each sum the row)
 template <typename T>
 __global__ void __launch_bounds__(512)
 window_intake_whole_kernel(IntakeArgs a, T* __restrict__ q_out, T* __restrict__ k_pages, T* __restrict__ v_pages) {
-  __shared__ float red[16];
+  __shared__ float red[2][8];
   const int wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE, n_waves = blockDim.x / SYN_WAVE;
   const int tok = blockIdx.x, nq = a.nh * a.dim, nk = a.write_kv ? a.nkv * a.dim : 0;
   const float* row = a.proj + (size_t)tok * a.width;
-  float sq = 0.f, sk = 0.f;
-  for (int d = threadIdx.x; d < nq + nk; d += blockDim.x) {
-    const float v = row[d] + (a.bias ? a.bias[d] : 0.f);
-    if (d < nq) sq = fmaf(v, v, sq);
-    else sk = fmaf(v, v, sk);
-  }
-  sq = block_sum(sq, red);
-  if (nk) sk = block_sum(sk, red);       // (the same for the whole workgroup)
+  // (eight loads of a thread under way at a time)
+  auto squares = [&](int from, int n) {
+    float s = 0.f;
+    for (int d0 = threadIdx.x; d0 < n; d0 += 8 * blockDim.x) {
+      float v[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int d = d0 + i * blockDim.x;
+        v[i] = d < n ? row[from + d] + (a.bias ? a.bias[from + d] : 0.f) : 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s = fmaf(v[i], v[i], s);
+    }
+    return s;
+  };
+  float sq = squares(0, nq), sk = squares(nq, nk);
+  sq = wave_sum(sq), sk = wave_sum(sk);
+  if (lane == 0) red[0][wave] = sq, red[1][wave] = sk;
+  __syncthreads();
+  sq = sk = 0.f;
+  for (int w = 0; w < n_waves; ++w) sq += red[0][w], sk += red[1][w];
   const float inv_q = 1.f / sqrtf(sq / (float)nq + a.eps), inv_k = nk ? 1.f / sqrtf(sk / (float)nk + a.eps) : 1.f;
   const int items = a.write_kv ? a.nh + a.nkv + a.nv : a.nh;
-  for (int item = wave; item < items; item += n_waves) {
+  for (int item = blockIdx.y * n_waves + wave; item < items; item += n_waves * gridDim.y) {
     const IntakeItem t = intake_item(a, item);
     const float* gain = t.is_q ? a.q_gain + item * a.dim : (t.is_k ? a.k_gain + (item - a.nh) * a.dim : nullptr);
     intake_store<T>(a, t, tok, item, lane, gain, t.is_q ? inv_q : inv_k, q_out, k_pages, v_pages);
@@ -193,8 +207,11 @@ SYN_EXPORT int syn_window_intake(const float* proj, int width, const float* bias
                         rot, pairs, nh, nkv, nv, dim, vdim, write_kv, values_are_keys ? nh * dim : (nh + nkv) * dim,
                         temp_coef, temp_every};
   if (norm_whole) {
-    if (is_f32) window_intake_whole_kernel<float><<<n_tokens, 512, 0, stream>>>(a, (float*)q_out, (float*)k_pages, (float*)v_pages);
-    else window_intake_whole_kernel<bf16><<<n_tokens, 512, 0, stream>>>(a, (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages);
+    // a token's items in one workgroup where the tokens fill the compute units, else spread over several
+    const int shares = max(1, min((items + 7) / 8, syn_compute_units() / n_tokens));
+    const dim3 whole(n_tokens, shares);
+    if (is_f32) window_intake_whole_kernel<float><<<whole, 512, 0, stream>>>(a, (float*)q_out, (float*)k_pages, (float*)v_pages);
+    else window_intake_whole_kernel<bf16><<<whole, 512, 0, stream>>>(a, (bf16*)q_out, (bf16*)k_pages, (bf16*)v_pages);
     SYN_LAUNCH_CHECK("window_intake_whole");
     return 0;
   }

@@ -216,6 +216,34 @@ __global__ void rmsnorm_rows_kernel(const T* __restrict__ x, size_t x_stride, co
     o[i] = from_f32<TOut>(load_gain(gain, gain_is_f32, i, gain_offset) * to_f32<T>(xr[i]) * inv);
 }
 
+// A workgroup a row, for rows wider than a few waves' worth: the values stay in registers (up to 8 a thread) between the
+// sum of squares and the scaling.
+#define RR_VPT 8
+template <typename T, typename TOut>
+__global__ void __launch_bounds__(256)
+rmsnorm_wide_rows_kernel(const T* __restrict__ x, size_t x_stride, const void* __restrict__ gain, int gain_is_f32,
+                         float gain_offset, float eps, TOut* __restrict__ out, int width) {
+  __shared__ float red[16];
+  const T* xr = x + (size_t)blockIdx.x * x_stride;
+  TOut* o = out + (size_t)blockIdx.x * width;
+  float v[RR_VPT], g[RR_VPT], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < RR_VPT; ++i) {
+    const int d = threadIdx.x + i * 256;
+    v[i] = d < width ? to_f32<T>(xr[d]) : 0.f;
+    g[i] = d < width ? load_gain(gain, gain_is_f32, d, gain_offset) : 0.f;
+  }
+#pragma unroll
+  for (int i = 0; i < RR_VPT; ++i) ss = fmaf(v[i], v[i], ss);
+  ss = block_sum(ss, red);
+  const float inv = rsqrtf(ss / (float)width + eps);
+#pragma unroll
+  for (int i = 0; i < RR_VPT; ++i) {
+    const int d = threadIdx.x + i * 256;
+    if (d < width) o[d] = from_f32<TOut>(g[i] * v[i] * inv);
+  }
+}
+
 SYN_EXPORT int syn_rmsnorm_rows(const void* x, int is_f32, long x_stride, const void* gain, int gain_is_f32,
                                 float gain_offset, float eps, void* out, int out_is_f32, int n_rows, int width,
                                 hipStream_t stream) {
@@ -223,9 +251,16 @@ SYN_EXPORT int syn_rmsnorm_rows(const void* x, int is_f32, long x_stride, const 
   SYN_CHECK(x_stride >= width && (is_f32 || !out_is_f32), "rmsnorm_rows: rows of %d values %ld apart", width, x_stride);
   const int wpb = 4;
   const int grid = (n_rows + wpb - 1) / wpb;
-#define SYN_RR(TIn, TOut)                                                                                                 \
-  rmsnorm_rows_kernel<TIn, TOut><<<grid, wpb * SYN_WAVE, 0, stream>>>((const TIn*)x, (size_t)x_stride, gain, gain_is_f32, \
-                                                                      gain_offset, eps, (TOut*)out, n_rows, width)
+  const bool wide = width > 256 && width <= RR_VPT * 256;
+#define SYN_RR(TIn, TOut)                                                                                                   \
+  do {                                                                                                                      \
+    if (wide)                                                                                                               \
+      rmsnorm_wide_rows_kernel<TIn, TOut><<<n_rows, 256, 0, stream>>>((const TIn*)x, (size_t)x_stride, gain, gain_is_f32,   \
+                                                                      gain_offset, eps, (TOut*)out, width);                 \
+    else                                                                                                                    \
+      rmsnorm_rows_kernel<TIn, TOut><<<grid, wpb * SYN_WAVE, 0, stream>>>((const TIn*)x, (size_t)x_stride, gain, gain_is_f32, \
+                                                                          gain_offset, eps, (TOut*)out, n_rows, width);     \
+  } while (0)
   if (!is_f32) SYN_RR(bf16, bf16);
   else if (out_is_f32) SYN_RR(float, float);
   else SYN_RR(float, bf16);

@@ -225,7 +225,7 @@ def test_gate_as_silu_behind_the_heads_norm():
 
 # ----------------------------------------------------------------------------- attention
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("nh,nk,D,every,rot", [(4, 2, 16, 16, 0), (6, 6, 12, 1, 0), (3, 1, 10, 61, 4), (8, 4, 64, 7, 0), (40, 8, 96, 64, 0)])
+@pytest.mark.parametrize("nh,nk,D,every,rot", [(4, 2, 16, 16, 0), (6, 6, 12, 1, 0), (3, 1, 10, 61, 4), (8, 4, 64, 7, 0), (40, 8, 96, 64, 0), (64, 4, 128, 30, 0)])
 def test_intake_with_norms_over_all_heads_a_temperature_and_keys_as_values(nh, nk, D, every, rot, dtype):
     """Norms over the whole query and the whole key projection (heads of unlike sizes: a norm a head would show), values
     that are the keys before their norm, a temperature that steps between the tokens; pages over a border."""
@@ -361,7 +361,7 @@ def test_one_far_key_among_hundreds(dtype):
 def test_norm_of_the_first_columns_of_longer_rows():
     from synaptix_amd.kernels import ops
     g = torch.Generator().manual_seed(6)
-    for N, D in ((1, 24), (9, 130), (300, 96)):
+    for N, D in ((1, 24), (9, 130), (300, 96), (8, 257), (5, 1536), (3, 2048), (2, 2100)):
         x, gain = randn(g, N, D + 11), 1.0 + 0.3 * randn(g, D)
         want = P.rms_norm(x[:, :D], gain, 1e-5)
         xd = dev(x)
