@@ -5,9 +5,10 @@ from .kamivik import KamivikConfig
 from .repolix import RepolixConfig
 from .nilepel import NilepelConfig
 from .pizunex import PizunexConfig
+from .sunosun import SunosunConfig
 from .registry import (Architecture, register_architecture, resolve_architecture, known_architectures,
                        load_config, read_config_json)
 
 __all__ = ["ConfigError", "Qwen3Config", "BizipelConfig", "KamivikConfig", "RepolixConfig", "NilepelConfig",
-           "PizunexConfig", "Architecture", "register_architecture", "resolve_architecture",
+           "PizunexConfig", "SunosunConfig", "Architecture", "register_architecture", "resolve_architecture",
            "known_architectures", "load_config", "read_config_json"]

@@ -33,6 +33,8 @@ struct WindowTerms {
   const float* sinks;    // [heads] or nullptr: the score of a key without a value in every softmax
   int chunk;             // 0: none
   int gate_per_head;     // the gate's rows hold one number a head (else one for each value)
+  int ldo;               // values from one token's results to the next (heads x vdim, or columns of longer rows)
+  float out_scale;       // a factor on the results
 };
 
 // the first key that the query at `pos` sees (kept first keys aside); it never falls as pos grows
@@ -358,14 +360,14 @@ window_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, 
         if (lane + i * SYN_WAVE < vdim) o[i] += f * part_o[w][lane + i * SYN_WAVE];
     }
   }
-  T* orow = out + ((size_t)tok * nh + head) * vdim;
+  T* orow = out + (size_t)tok * terms.ldo + (size_t)head * vdim;
   const int per_head = terms.gate_per_head;
   const float* g = gate ? gate + (size_t)tok * gate_stride + (per_head ? head : (size_t)head * vdim) : nullptr;
 #pragma unroll
   for (int i = 0; i < MAXD / SYN_WAVE; ++i) {
     const int d = lane + i * SYN_WAVE;
     if (d < vdim) {
-      float v = o[i] / l;
+      float v = o[i] / l * terms.out_scale;
       if (g) {
         const float z = g[per_head ? 0 : d] + (gate_bias ? gate_bias[per_head ? head : head * vdim + d] : 0.f);
         v *= 1.f / (1.f + expf(-z));
@@ -381,8 +383,9 @@ SYN_EXPORT int syn_window_attention(const void* q, const void* k_pages, const vo
                                     const float* gate, int gate_stride, const float* gate_bias, void* out, float scale,
                                     int n_tokens, int nh, int nkv, int dim, int vdim, const float* slopes,
                                     const float* r1, const float* r2, float softcap, int window, int keep_first,
-                                    int sink_one, int v_share, const float* sinks, int chunk, int gate_per_head,
-                                    hipStream_t stream) {
+                                    int sink_one, int v_share, const float* sinks, int chunk, int gate_per_head, int ldo,
+                                    float out_scale, hipStream_t stream) {
+  SYN_CHECK(ldo >= nh * vdim, "window_attention: result rows of %d values", ldo);
   SYN_CHECK(n_tokens > 0 && nh > 0 && nkv > 0, "window_attention: empty input");
   SYN_CHECK(chunk >= 0 && !(sinks && sink_one), "window_attention: chunks of %d, or two sinks", chunk);
   SYN_CHECK(v_share > 0 && nkv % v_share == 0, "window_attention: %d kv heads in shares of %d", nkv, v_share);
@@ -394,7 +397,7 @@ SYN_EXPORT int syn_window_attention(const void* q, const void* k_pages, const vo
   SYN_CHECK((r1 == nullptr) == (r2 == nullptr), "window_attention: r1 and r2 come together");
   SYN_CHECK(gate == nullptr || gate_stride >= (gate_per_head ? nh : nh * vdim), "window_attention: gate rows of %d values",
             gate_stride);
-  const WindowTerms terms = {slopes, r1, r2, softcap, window, keep_first, sink_one, v_share, sinks, chunk, gate_per_head};
+  const WindowTerms terms = {slopes, r1, r2, softcap, window, keep_first, sink_one, v_share, sinks, chunk, gate_per_head, ldo, out_scale};
   const dim3 grid(n_tokens, nh);
   // few (token, head) pairs (single tokens of a few sequences): eight waves share each pair's keys
   const bool many_waves = (long)n_tokens * nh < 8L * syn_compute_units();
@@ -632,7 +635,7 @@ window_prefill_bf16_kernel(const bf16* __restrict__ q, const bf16* __restrict__ 
     }
   }
   if (!q_ok) return;
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv = l > 0.f ? terms.out_scale / l : 0.f;
   const size_t tok = (size_t)(start + my_n);
 #pragma unroll
   for (int j = 0; j < AWP_TILES; ++j) {
@@ -649,7 +652,7 @@ window_prefill_bf16_kernel(const bf16* __restrict__ q, const bf16* __restrict__ 
         }
         o4[e] = (bf16)v;
       }
-      *(bf16x4*)(out + tok * nh * vdim + col) = o4;
+      *(bf16x4*)(out + tok * terms.ldo + col) = o4;
     }
   }
 }
@@ -662,8 +665,9 @@ SYN_EXPORT int syn_window_attention_prefill_bf16(const void* q, const void* k_pa
                                                  int gate_stride, const float* gate_bias, void* out, float scale, int nh,
                                                  int nkv, int dim, int vdim, const float* slopes, const float* r1,
                                                  const float* r2, float softcap, int window, int keep_first, int sink_one,
-                                                 int v_share, const float* sinks, int chunk, int gate_per_head,
-                                                 hipStream_t stream) {
+                                                 int v_share, const float* sinks, int chunk, int gate_per_head, int ldo,
+                                                 float out_scale, hipStream_t stream) {
+  SYN_CHECK(ldo >= nh * vdim && ldo % 4 == 0, "window_attention_prefill: result rows of %d values (a multiple of 4)", ldo);
   SYN_CHECK(n_tokens > 0 && n_seqs > 0 && nh > 0 && nkv > 0, "window_attention_prefill: empty input");
   SYN_CHECK(v_share > 0 && nkv % v_share == 0, "window_attention_prefill: %d kv heads in shares of %d", nkv, v_share);
   SYN_CHECK(nh % nkv == 0, "window_attention_prefill: %d heads do not divide into %d kv heads", nh, nkv);
@@ -677,7 +681,7 @@ SYN_EXPORT int syn_window_attention_prefill_bf16(const void* q, const void* k_pa
   SYN_CHECK(chunk >= 0 && !(sinks && sink_one), "window_attention_prefill: chunks of %d, or two sinks", chunk);
   SYN_CHECK((uintptr_t)q % 16 == 0 && (uintptr_t)k_pages % 16 == 0 && (uintptr_t)v_pages % 16 == 0 && (uintptr_t)out % 8 == 0,
             "window_attention_prefill: operands are not aligned");
-  const WindowTerms terms = {slopes, r1, r2, softcap, window, keep_first, sink_one, v_share, sinks, chunk, gate_per_head};
+  const WindowTerms terms = {slopes, r1, r2, softcap, window, keep_first, sink_one, v_share, sinks, chunk, gate_per_head, ldo, out_scale};
   const dim3 grid((n_tokens + 63) / 64 + n_seqs, nh);      // at most this many tiles of 64 queries; the rest leave at once
   if (dim % 32 == 0)
     window_prefill_bf16_kernel<true><<<grid, 256, 0, stream>>>(

@@ -134,6 +134,7 @@ __device__ __forceinline__ float gated(int act, float gate, float up, float limi
 #define SYN_POINT_NONE 0
 #define SYN_POINT_RELU_SQUARED 1
 #define SYN_POINT_COUNT 2
+#define SYN_POINT_SOFTCAP 2     // cap * tanh(z / cap) on an output head's logits: only the products for few rows have it
 __device__ __forceinline__ float point_activation(int point, float z) {
   if (point == SYN_POINT_RELU_SQUARED) {
     z = z > 0.f ? z : (z <= 0.f ? 0.f : z);      // (a NaN stays one)
@@ -141,6 +142,7 @@ __device__ __forceinline__ float point_activation(int point, float z) {
   }
   return z;
 }
+__device__ __forceinline__ float soft_cap(float z, float cap) { return cap * tanhf(z / cap); }
 
 // ---- what an attention kernel may do to a scaled score before the mask and the softmax ----
 // A soft cap, cap * tanh(score / cap), and a penalty in the distance between query and key, - slope[head] * (q - k)

@@ -13,41 +13,67 @@ SYN_DEFINE_ERROR_CHANNEL
 
 // ------------------------------------------------------------------ embedding
 // resid[n, :] = scale * table[ids[n], :] widened to float.  Ids are checked on the host.
+// pos.rates != null: a sinusoidal position vector is added, sin(p f_i) at column 2 i and cos(p f_i) at 2 i + 1 for the token
+// at position p; the angle is taken in 64-bit and reduced to one turn there, so that it is as good at any position as near 0.
+// keep != null: the rows once more (resid is written on by the layers).
+struct EmbedPositions {
+  const double* rates;   // [(H + 1) / 2] f_i, or null
+  const int* pos;        // [tokens]
+};
+__device__ __forceinline__ float embed_position(const EmbedPositions& p, int n, int col) {
+  constexpr double TURN = 6.283185307179586;
+  double a = (double)p.pos[n] * p.rates[col / 2];
+  a -= TURN * rint(a / TURN);
+  return col % 2 ? cosf((float)a) : sinf((float)a);
+}
+
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ ids, float* __restrict__ resid,
-                             int H, float scale) {
+                             int H, float scale, EmbedPositions p, float* __restrict__ keep) {
   const int n = blockIdx.x;
   const T* row = table + (size_t)ids[n] * H;
   float* out = resid + (size_t)n * H;
-  for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = to_f32<T>(row[i]) * scale;
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    float v = to_f32<T>(row[i]) * scale;
+    if (p.rates) v += embed_position(p, n, i);
+    out[i] = v;
+    if (keep) keep[(size_t)n * H + i] = v;
+  }
 }
 
 // the same from a bf16 table in fragment order ([V / 16][H / 32][64 lanes][8], as the products read the tied
 // output head): eight consecutive values of a row are one lane's 16 bytes
 __global__ void embed_packed_kernel(const bf16* __restrict__ table, const int* __restrict__ ids, float* __restrict__ resid,
-                                    int H, float scale) {
+                                    int H, float scale, EmbedPositions p, float* __restrict__ keep) {
   const int n = blockIdx.x, id = ids[n];
   const bf16* group = table + (size_t)(id / 16) * H * 16;   // the 16 rows around row id: H / 32 fragments of 512 values
   float* out = resid + (size_t)n * H;
   for (int c = threadIdx.x; c < H / 8; c += blockDim.x) {   // chunk c: values 8 c .. 8 c + 7 of the row
     const bf16x8 v = *(const bf16x8*)(group + (size_t)(c / 4) * 512 + ((c % 4) * 16 + id % 16) * 8);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) out[c * 8 + e] = (float)v[e] * scale;
+    for (int e = 0; e < 8; ++e) {
+      float x = (float)v[e] * scale;
+      if (p.rates) x += embed_position(p, n, c * 8 + e);
+      out[c * 8 + e] = x;
+      if (keep) keep[(size_t)n * H + c * 8 + e] = x;
+    }
   }
 }
 
 // table_kind: 0 = bf16 rows, 1 = float rows, 2 = bf16 in fragment order (V a multiple of 16, H of 32)
 SYN_EXPORT int syn_embed(const void* table, int table_kind, const int* ids, float* resid, int n_tokens, int H,
-                         float scale, hipStream_t stream) {
+                         float scale, const double* rates, const int* pos, float* keep, hipStream_t stream) {
+  SYN_CHECK((rates == nullptr) == (pos == nullptr), "embed: rates and positions come together");
+  const EmbedPositions p = {rates, pos};
   SYN_CHECK(n_tokens > 0 && H > 0, "embed: empty input (%d tokens, width %d)", n_tokens, H);
   SYN_CHECK(table_kind >= 0 && table_kind <= 2, "embed: unknown kind of table %d", table_kind);
   if (table_kind == 1) {
-    embed_kernel<float><<<n_tokens, 256, 0, stream>>>((const float*)table, ids, resid, H, scale);
+    embed_kernel<float><<<n_tokens, 256, 0, stream>>>((const float*)table, ids, resid, H, scale, p, keep);
   } else if (table_kind == 2) {
     SYN_CHECK(H % 32 == 0, "embed: a table in fragment order has a width that is a multiple of 32, not %d", H);
-    embed_packed_kernel<<<n_tokens, 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale);
+    embed_packed_kernel<<<n_tokens, 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale, p, keep);
   } else {
-    embed_kernel<bf16><<<n_tokens, 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale);
+    embed_kernel<bf16><<<n_tokens, 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale, p, keep);
   }
   SYN_LAUNCH_CHECK("embed");
   return 0;
@@ -685,15 +711,17 @@ SYN_EXPORT int syn_qk_norm_rope_kv_write(const void* qkv, int n_parts, void* q_o
 // A layer whose sublayers run side by side on one normed input leaves up to two results, each with a scale of its
 // own for every channel:   x[r] += s1 * d1[r] + s2 * d2[r]   (s: float [H], d: n_parts partial sums [parts][rows][H]
 // added in order, or null), then out[r] = norm(x[r]) * gain if `out` is given.  A term may also carry a gate for every
-// row (g: one float a row at g[r * stride], or null): the term is then multiplied by sigmoid(g[r]).  With `rows` only those rows are summed
+// row (g: one float a row at g[r * stride], or null): the term is then multiplied by sigmoid(g[r]).  add_rows [rows][H] and
+// add_vec [H] (or null) are added beside the terms.  With `rows` only those rows are summed
 // and normed, and x stays as it is.  32-bit throughout; one rounding at the store.
 template <typename TOut>
 __global__ void add_scaled_rmsnorm_kernel(float* __restrict__ resid, const int* __restrict__ rows, size_t part_stride,
                                           const float* __restrict__ d1, int parts1, const float* __restrict__ s1,
                                           const float* __restrict__ d2, int parts2, const float* __restrict__ s2,
                                           const float* __restrict__ g1, int g1_stride, const float* __restrict__ g2,
-                                          int g2_stride, const void* __restrict__ gain, int gain_is_f32, float eps,
-                                          TOut* __restrict__ out, int H) {
+                                          int g2_stride, const float* __restrict__ add_rows,
+                                          const float* __restrict__ add_vec, const void* __restrict__ gain,
+                                          int gain_is_f32, float eps, TOut* __restrict__ out, int H) {
   __shared__ float red[16];
   const int r = rows ? rows[blockIdx.x] : blockIdx.x;
   // a term's factor for the whole row: the sigmoid of one number a row (or 1)
@@ -715,6 +743,8 @@ __global__ void add_scaled_rmsnorm_kernel(float* __restrict__ resid, const int* 
       for (int p = 0; p < parts2; ++p) t += b[p * part_stride + i];
       v = fmaf(s2 ? s2[i] * f2 : f2, t, v);
     }
+    if (add_rows) v += add_rows[(size_t)r * H + i];
+    if (add_vec) v += add_vec[i];
     return v;
   };
   float ss = 0.f;
@@ -735,7 +765,8 @@ __global__ void add_scaled_rmsnorm_kernel(float* __restrict__ resid, const int* 
 
 SYN_EXPORT int syn_add_scaled_rmsnorm(float* resid, int n_rows, const int* rows, int n_out, const float* d1, int parts1,
                                       const float* s1, const float* d2, int parts2, const float* s2, const float* g1,
-                                      int g1_stride, const float* g2, int g2_stride, const void* gain,
+                                      int g1_stride, const float* g2, int g2_stride, const float* add_rows,
+                                      const float* add_vec, const void* gain,
                                       int gain_is_f32, float eps, void* out, int out_is_f32, int H, hipStream_t stream) {
   SYN_CHECK(n_out > 0 && H > 0 && n_rows > 0, "add_scaled_rmsnorm: empty input (%d rows, width %d)", n_out, H);
   SYN_CHECK(parts1 >= 1 && parts1 <= 64 && parts2 >= 1 && parts2 <= 64, "add_scaled_rmsnorm: %d and %d partial sums", parts1, parts2);
@@ -744,12 +775,25 @@ SYN_EXPORT int syn_add_scaled_rmsnorm(float* resid, int n_rows, const int* rows,
   const int block = H >= 4096 ? 1024 : (H >= 1024 ? 512 : 256);
   if (out_is_f32)
     add_scaled_rmsnorm_kernel<float><<<n_out, block, 0, stream>>>(resid, rows, stride, d1, parts1, s1, d2, parts2, s2, g1,
-                                                                  g1_stride, g2, g2_stride, gain,
+                                                                  g1_stride, g2, g2_stride, add_rows, add_vec, gain,
                                                                   gain_is_f32, eps, (float*)out, H);
   else
     add_scaled_rmsnorm_kernel<bf16><<<n_out, block, 0, stream>>>(resid, rows, stride, d1, parts1, s1, d2, parts2, s2, g1,
-                                                                  g1_stride, g2, g2_stride, gain,
+                                                                  g1_stride, g2, g2_stride, add_rows, add_vec, gain,
                                                                  gain_is_f32, eps, (bf16*)out, H);
   SYN_LAUNCH_CHECK("add_scaled_rmsnorm");
+  return 0;
+}
+
+// ------------------------------------------------------------------ soft cap, in place
+__global__ void soft_cap_kernel(float* __restrict__ x, size_t n, float cap) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) x[i] = soft_cap(x[i], cap);
+}
+
+SYN_EXPORT int syn_soft_cap(float* x, long n, float cap, hipStream_t stream) {
+  SYN_CHECK(n > 0 && cap > 0.f, "soft_cap: %ld values, cap %g", n, (double)cap);
+  soft_cap_kernel<<<(n + 255) / 256, 256, 0, stream>>>(x, (size_t)n, cap);
+  SYN_LAUNCH_CHECK("soft_cap");
   return 0;
 }

@@ -194,6 +194,8 @@ struct RowNorm {
   const void* gain;   // [N] bf16 or float
   int gain_is_f32;
   float gain_offset;
+  const float* add_rows;   // [M, N] or null: what else the residual rows get (parts.linear.InjectedDelta)
+  const float* add_vec;    // [N] or null: the same for every row
 };
 
 // inv[m] for the rows of x into LDS (16 floats): wave w takes rows w and w + n_waves (up to 16 rows, 8 waves or more).
@@ -243,6 +245,11 @@ __device__ __forceinline__ void resid_norm_store(const RowNorm& rn, bool in, int
   if (in && (n & 15) == 0) rn.ss_out[(size_t)m * (N / 16) + n / 16] = q;
 }
 
+// what the sums of the products for few rows may pass before they are stored: the points of every product, and a soft cap
+__device__ __forceinline__ float packed_point(const Epilogue& ep, float v) {
+  return ep.point == SYN_POINT_SOFTCAP ? soft_cap(v, ep.limit) : point_activation(ep.point, v);
+}
+
 // ------------------------------------------------------------------ few rows of x, W in fragment order
 // The same scheme as gemm_skinny (up to 16 rows of x, K split over the waves of a group, partial
 // tiles summed in LDS in a fixed order) over a copy of W that is kept in the order of the MFMA
@@ -280,7 +287,11 @@ gemm_packed_kernel(const bf16* __restrict__ x, const bf16* __restrict__ wp, void
   if (!PAIRED && rn.resid && threadIdx.x < TILES * 256) {
     const int t = threadIdx.x / 256, j = (threadIdx.x / 64) % 4, ln = threadIdx.x % 64;
     const int m = 4 * (ln / 16) + j, n = ((int)blockIdx.x * TILES + t) * 16 + ln % 16;
-    if (m < M && n < N) r0 = rn.resid[(size_t)m * N + n], g0 = load_gain(rn.gain, rn.gain_is_f32, n, rn.gain_offset);
+    if (m < M && n < N) {
+      r0 = rn.resid[(size_t)m * N + n], g0 = load_gain(rn.gain, rn.gain_is_f32, n, rn.gain_offset);
+      if (rn.add_rows) r0 += rn.add_rows[(size_t)m * N + n];
+      if (rn.add_vec) r0 += rn.add_vec[n];
+    }
   }
   // blockIdx.y = which slice of K (ks_slice k-steps of 32) this workgroup sums; its output is slice blockIdx.y
   // of a float [slices, M, N] that the reader adds up (a product with few rows of W gets more workgroups so)
@@ -328,7 +339,7 @@ gemm_packed_kernel(const bf16* __restrict__ x, const bf16* __restrict__ wp, void
       if (rn.resid) {   // the same for the whole workgroup
         resid_norm_store(rn, in, m, n, N, v, r0, g0);
       } else if (in) {
-        v = point_activation(ep.point, v);
+        v = packed_point(ep, v);
         if (ep.out_is_f32)
           ((float*)out)[((size_t)blockIdx.y * M + m) * N + n] = v;
         else
@@ -411,7 +422,7 @@ gemm_packed2_kernel(const bf16* __restrict__ x, const bf16* __restrict__ wp, voi
       if (m < M && n < N && (t == 0 || second)) {
         float v = summed(t, j, ln);
         if (rn.ss) v *= inv[m];
-        v = point_activation(ep.point, v);
+        v = packed_point(ep, v);
         if (ep.out_is_f32) ((float*)out)[((size_t)blockIdx.y * M + m) * N + n] = v;
         else ((bf16*)out)[(size_t)m * N + n] = (bf16)v;
       }
@@ -1175,14 +1186,17 @@ SYN_EXPORT int syn_gemm_swiglu(const void* x, const void* w, void* out, int M, i
 //   ss [M, ss_groups] float (or null): the sums of row m are multiplied by rsqrt(sum(ss[m, :]) / norm_dim + eps);
 //   resid [M, N] float (or null; then float sums, one slice, not paired, `out` unused): resid += sums,
 //   xs [M, N] bf16 = (gain_offset + gain[n]) * resid, ss_out [M, N / 16] = sums of resid^2 over groups of 16 columns.
-// point: as for syn_gemm.
+// point: as for syn_gemm, or SYN_POINT_SOFTCAP with its cap in `limit`.
+// add_rows [M, N], add_vec [N] (or null): added into resid beside the sums.
 SYN_EXPORT int syn_gemm_packed_norm(const void* x, const void* wp, void* out, int out_code, int M, int N, int K, int paired,
                                     int act, float limit, int slices, const float* ss, int ss_groups, int norm_dim, float eps,
                                     float* resid, void* xs, float* ss_out, const void* gain, int gain_is_f32,
-                                    float gain_offset, int point, hipStream_t stream) {
-  SYN_CHECK(point >= 0 && point < SYN_POINT_COUNT && (point == SYN_POINT_NONE || (slices == 1 && !paired && !resid)),
+                                    float gain_offset, const float* add_rows, const float* add_vec, int point,
+                                    hipStream_t stream) {
+  SYN_CHECK(point >= 0 && point <= SYN_POINT_SOFTCAP && (point == SYN_POINT_NONE || (slices == 1 && !paired && !resid)),
             "gemm_packed: activation code %d belongs to a plain product in one slice", point);
   SYN_CHECK(act >= 0 && act < SYN_ACT_COUNT, "gemm_packed: unknown activation code %d", act);
+  SYN_CHECK(point != SYN_POINT_SOFTCAP || limit > 0.f, "gemm_packed: a soft cap of %g", (double)limit);
   SYN_CHECK(slices >= 1 && slices <= 64 && (slices == 1 || (out_code == 2 && !paired)),
             "gemm_packed: %d slices of K need a float output [slices, M, N] and no activation", slices);
   const Epilogue ep = {out_code == 2, act, limit, point};
@@ -1201,7 +1215,7 @@ SYN_EXPORT int syn_gemm_packed_norm(const void* x, const void* wp, void* out, in
     SYN_CHECK(!paired && slices == 1 && out_code == 2 && xs && ss_out && gain,
               "gemm_packed: the product before a norm is one slice of float sums with xs, ss_out and a gain");
     rn.resid = resid, rn.xs = (bf16*)xs, rn.ss_out = ss_out, rn.gain = gain, rn.gain_is_f32 = gain_is_f32;
-    rn.gain_offset = gain_offset;
+    rn.gain_offset = gain_offset, rn.add_rows = add_rows, rn.add_vec = add_vec;
   }
   const bf16* xb = (const bf16*)x;
   const bf16* wb = (const bf16*)wp;
@@ -1225,5 +1239,5 @@ SYN_EXPORT int syn_gemm_packed_norm(const void* x, const void* wp, void* out, in
 SYN_EXPORT int syn_gemm_packed(const void* x, const void* wp, void* out, int out_code, int M, int N, int K, int paired,
                                int act, float limit, int slices, int point, hipStream_t stream) {
   return syn_gemm_packed_norm(x, wp, out, out_code, M, N, K, paired, act, limit, slices, nullptr, 0, 0, 0.f, nullptr, nullptr,
-                              nullptr, nullptr, 0, 0.f, point, stream);
+                              nullptr, nullptr, 0, 0.f, nullptr, nullptr, point, stream);
 }

@@ -7,7 +7,7 @@
 //     arow(r) = a_rows[r] and orow(r) = o_rows[r] gathered through index lists;
 //   * every group takes all M rows (a linear map for each head of a token): A, W and out move on by a fixed
 //     number of elements from one group to the next.
-// Epilogue, in this order and each optional: the exact GELU 0.5 z (1 + erf(z / sqrt 2)); a weight of the row;
+// Epilogue, in this order and each optional: the exact GELU 0.5 z (1 + erf(z / sqrt 2)) or max(z, 0)^2; a weight of the row;
 // sigmoid of a gate value read from float rows.  Or, with `pair`: W's rows come in pairs (2 j: the gate row of output j,
 // 2 j + 1: its up row) and what is stored is the gated activation of the two sums (gated, csrc/common.h), N / 2 columns.  Sums are 32-bit.  bf16 operands whose K is a multiple of 32 run on
 // the matrix cores: with few rows a group 16x16x32 with operands straight from memory as 16-byte pieces of rows (no
@@ -33,7 +33,7 @@ struct GroupedArgs {
   const float* gate;        // or null: gate[row * gate_ld + group * gate_group + n * gate_col]
   long gate_ld, gate_group;
   int gate_col;
-  int act;                  // 0: none, 1: exact GELU
+  int act;                  // 0: none, 1: exact GELU, 2: max(z, 0)^2
   int pair;                 // 0: none; else 1 + the code of the gated activation over pairs of rows of W
   float limit;              // that activation's bound, if it has one
   int M, N, K, groups;
@@ -50,6 +50,7 @@ __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.f + er
 
 __device__ __forceinline__ float grouped_epilogue(const GroupedArgs& g, float v, int r, int b, int n) {
   if (g.act == 1) v = gelu_erf(v);
+  if (g.act == 2) v = point_activation(SYN_POINT_RELU_SQUARED, v);
   if (g.row_weight) v *= g.row_weight[r];
   if (g.gate) {
     const float z = g.gate[(size_t)r * g.gate_ld + (size_t)b * g.gate_group + (size_t)n * g.gate_col];
@@ -365,7 +366,7 @@ SYN_EXPORT int syn_grouped_product(const void* a, long lda, long a_group, const 
                                    int rows_bound, int force_simt, int w_packed, int pair, float limit,
                                    hipStream_t stream) {
   SYN_CHECK(M > 0 && N > 0 && K > 0 && groups > 0, "grouped_product: empty input (%d rows, %d x %d, %d groups)", M, N, K, groups);
-  SYN_CHECK(act == 0 || act == 1, "grouped_product: unknown activation code %d", act);
+  SYN_CHECK(act >= 0 && act <= 2, "grouped_product: unknown activation code %d", act);
   SYN_CHECK(pair >= 0 && pair <= SYN_ACT_COUNT && (pair == 0 || (N % 2 == 0 && act == 0 && gate == nullptr)),
             "grouped_product: a gated activation (code %d) over %d rows of W in pairs, with no other activation", pair - 1, N);
   SYN_CHECK(seg_start != nullptr || (a_rows == nullptr && o_rows == nullptr && row_weight == nullptr),
@@ -477,15 +478,16 @@ SYN_EXPORT int syn_route_topk(const float* logits, const float* bias, int* ids, 
 }
 
 // ---------------------------------------------------------------- a router that scores all experts
-// s = softmax(logits) over all E outputs (32-bit).  The choice is made on s + correction: the E outputs form n_groups
-// equal groups of neighbours, a group's score is its largest choice score, only members of the keep_groups best groups
+// s = softmax(logits) over all E outputs, or, with `sigmoid`, the sigmoid of each (32-bit).  The choice is made on
+// s + correction: the E outputs form n_groups equal groups of neighbours, a group's score is its largest choice score, or,
+// with group_two, the sum of its two largest; only members of the keep_groups best groups
 // can be chosen (the others count as minus infinity), and of those the `top` largest are taken (the lower index of
 // equal ones, for groups and for experts).  weights: the chosen experts' s itself, without the correction; renorm:
-// divided by their sum.  One wave a token.
+// divided by their sum (+ renorm_eps).  One wave a token.
 __global__ void __launch_bounds__(256) route_scores_kernel(const float* __restrict__ logits, const float* __restrict__ correction,
                                                            int* __restrict__ ids, float* __restrict__ weights, int n_tokens,
                                                            int E, int ld, int top, int n_groups, int keep_groups, int renorm,
-                                                           float scale) {
+                                                           float scale, int sigmoid, int group_two, float renorm_eps) {
   __shared__ float ss[4][ROUTE_MAX_EXPERTS];       // the scores
   __shared__ float cs[4][ROUTE_MAX_EXPERTS];       // the choice scores
   __shared__ float gs[4][ROUTE_MAX_EXPERTS];       // the groups' scores
@@ -501,16 +503,21 @@ __global__ void __launch_bounds__(256) route_scores_kernel(const float* __restri
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   };
-  float mx = -INFINITY;
-  for (int e = lane; e < E; e += SYN_WAVE) mx = fmaxf(mx, logits[(size_t)tok * ld + e]);
-  mx = wave_max(mx);
-  float sum = 0.f;
-  for (int e = lane; e < E; e += SYN_WAVE) {
-    const float p = expf(logits[(size_t)tok * ld + e] - mx);
-    sc[e] = p;
-    sum += p;
+  float sum = 1.f;
+  if (sigmoid) {
+    for (int e = lane; e < E; e += SYN_WAVE) sc[e] = 1.f / (1.f + expf(-logits[(size_t)tok * ld + e]));
+  } else {
+    float mx = -INFINITY;
+    for (int e = lane; e < E; e += SYN_WAVE) mx = fmaxf(mx, logits[(size_t)tok * ld + e]);
+    mx = wave_max(mx);
+    sum = 0.f;
+    for (int e = lane; e < E; e += SYN_WAVE) {
+      const float p = expf(logits[(size_t)tok * ld + e] - mx);
+      sc[e] = p;
+      sum += p;
+    }
+    sum = wave_sum(sum);
   }
-  sum = wave_sum(sum);
   const int per = E / n_groups;
   for (int e = lane; e < E; e += SYN_WAVE) {
     sc[e] = sc[e] / sum;
@@ -519,9 +526,13 @@ __global__ void __launch_bounds__(256) route_scores_kernel(const float* __restri
   wave_sync();
   if (keep_groups < n_groups) {
     for (int g = lane; g < n_groups; g += SYN_WAVE) {
-      float best = -INFINITY;
-      for (int j = 0; j < per; ++j) best = fmaxf(best, c[g * per + j]);
-      grp[g] = best;
+      float best = -INFINITY, second = -INFINITY;
+      for (int j = 0; j < per; ++j) {
+        const float v = c[g * per + j];
+        second = fmaxf(second, fminf(best, v));
+        best = fmaxf(best, v);
+      }
+      grp[g] = group_two && per > 1 ? best + second : best;
     }
     wave_sync();
     // a group stays if fewer than keep_groups others come before it (a larger score, or an equal one at a lower index)
@@ -559,6 +570,7 @@ __global__ void __launch_bounds__(256) route_scores_kernel(const float* __restri
     if (renorm) {
       total = 0.f;
       for (int t = 0; t < top; ++t) total += chosen[t];
+      total += renorm_eps;
     }
     for (int t = 0; t < top; ++t) weights[(size_t)tok * top + t] = chosen[t] / total * scale;
   }
@@ -567,7 +579,8 @@ __global__ void __launch_bounds__(256) route_scores_kernel(const float* __restri
 // logits: rows of `ld` values whose first E are the router's outputs; weights: the chosen scores (over their sum with
 // renorm) times `scale`
 SYN_EXPORT int syn_route_scores(const float* logits, const float* correction, int* ids, float* weights, int n_tokens, int E,
-                                int ld, int top, int n_groups, int keep_groups, int renorm, float scale, hipStream_t stream) {
+                                int ld, int top, int n_groups, int keep_groups, int renorm, float scale, int sigmoid, int group_two,
+                                float renorm_eps, hipStream_t stream) {
   SYN_CHECK(ld >= E, "route_scores: rows of %d values for %d experts", ld, E);
   SYN_CHECK(n_tokens > 0, "route_scores: empty input");
   SYN_CHECK(E > 0 && E <= ROUTE_MAX_EXPERTS, "route_scores: %d experts (at most %d)", E, ROUTE_MAX_EXPERTS);
@@ -576,7 +589,7 @@ SYN_EXPORT int syn_route_scores(const float* logits, const float* correction, in
   SYN_CHECK(top > 0 && top <= ROUTE_MAX_TOP && top <= keep_groups * (E / n_groups),
             "route_scores: the %d largest of %d groups of %d (at most %d)", top, keep_groups, E / n_groups, ROUTE_MAX_TOP);
   route_scores_kernel<<<(n_tokens + 3) / 4, 256, 0, stream>>>(logits, correction, ids, weights, n_tokens, E, ld, top, n_groups,
-                                                             keep_groups, renorm, scale);
+                                                             keep_groups, renorm, scale, sigmoid, group_two, renorm_eps);
   SYN_LAUNCH_CHECK("route_scores");
   return 0;
 }

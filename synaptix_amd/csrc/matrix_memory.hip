@@ -515,7 +515,7 @@ SYN_EXPORT int syn_matrix_memory_scan(const float* proj, int width, const float*
 template <typename TOut>
 __global__ void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ gain, float eps,
                                       const float* __restrict__ gate, int gate_stride, TOut* __restrict__ out,
-                                      int n_items, int H, int vdim, int kind) {
+                                      int out_stride, int n_items, int H, int vdim, int kind) {
   const int item = blockIdx.x * (blockDim.x / SYN_WAVE) + threadIdx.x / SYN_WAVE;
   if (item >= n_items) return;
   const int lane = threadIdx.x % SYN_WAVE;
@@ -533,23 +533,24 @@ __global__ void head_norm_gate_kernel(const float* __restrict__ o, const float* 
     float v = (first ? x[d] * (g[d] / (1.f + expf(-g[d]))) : x[d]) * inv;
     if (gain) v *= gain[h * vdim + d];
     if (g && !first) v *= (kind == HNG_SILU ? g[d] : 1.f) / (1.f + expf(-g[d]));
-    out[((size_t)tok * H + h) * vdim + d] = from_f32<TOut>(v);
+    out[(size_t)tok * out_stride + (size_t)h * vdim + d] = from_f32<TOut>(v);
   }
 }
 
 SYN_EXPORT int syn_head_norm_gate(const float* o, const float* gain, float eps, const float* gate, int gate_stride,
-                                  void* out, int out_is_f32, int n_tokens, int H, int vdim, int kind,
+                                  void* out, int out_stride, int out_is_f32, int n_tokens, int H, int vdim, int kind,
                                   hipStream_t stream) {
   SYN_CHECK(n_tokens > 0 && H > 0 && vdim > 0, "head_norm_gate: empty input");
   SYN_CHECK(gate == nullptr || gate_stride >= H * vdim, "head_norm_gate: gate rows of %d values", gate_stride);
+  SYN_CHECK(out_stride >= H * vdim, "head_norm_gate: result rows of %d values", out_stride);
   SYN_CHECK(kind >= HNG_SIGMOID && kind <= HNG_SILU, "head_norm_gate: unknown kind of gate %d", kind);
   const int wpb = 4, items = n_tokens * H;
   const int grid = (items + wpb - 1) / wpb;
   if (out_is_f32)
-    head_norm_gate_kernel<float><<<grid, wpb * SYN_WAVE, 0, stream>>>(o, gain, eps, gate, gate_stride, (float*)out, items,
+    head_norm_gate_kernel<float><<<grid, wpb * SYN_WAVE, 0, stream>>>(o, gain, eps, gate, gate_stride, (float*)out, out_stride, items,
                                                                       H, vdim, kind);
   else
-    head_norm_gate_kernel<bf16><<<grid, wpb * SYN_WAVE, 0, stream>>>(o, gain, eps, gate, gate_stride, (bf16*)out, items,
+    head_norm_gate_kernel<bf16><<<grid, wpb * SYN_WAVE, 0, stream>>>(o, gain, eps, gate, gate_stride, (bf16*)out, out_stride, items,
                                                                      H, vdim, kind);
   SYN_LAUNCH_CHECK("head_norm_gate");
   return 0;

@@ -7,6 +7,8 @@
 //   channel_delta_scan a decay for every key channel and the delta rule:
 //                      S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q                 (S: D x P)
 //   head_delta_scan    the same with one decay a head, S <- g S (prompts in chunks on the matrix cores)
+//   gated_linear_scan  a decay for every key channel, no correction: S <- diag(g) S + k v^T,  o = S^T q   (S: D x P; prompts in
+//                      chunks on the matrix cores), gated_linear_step: single tokens, with the heads' norm and gate
 //   diff_heads         two softmax maps over the same values, o = rms_norm(a1 - lambda a2) (1 - c)
 //
 // Everything here is 32-bit FMA: inputs are the float sums of the projections, states are float.  The scans walk a
@@ -863,6 +865,406 @@ SYN_EXPORT int syn_head_delta_scan(const float* qkv, const float* beta, int beta
 #undef SYN_HD2
 #undef SYN_HD
   SYN_LAUNCH_CHECK("head_delta_carry");
+  return 0;
+}
+
+// ---------------------------------------------------------------- gated linear attention
+//   z = A2 mid + bias (heads x D),  g = sigmoid(z)^(1 / tau) = exp(-softplus(-z) / tau);   S <- diag(g) S + k v^T,  o = S^T q
+// q, k, v and mid (the narrow middle W_a1 h in front of the decays' second product) are columns of one projection's rows.
+struct GlaArgs {
+  const float* q;
+  const float* k;
+  const float* v;
+  const float* mid;
+  int ld;                    // from one token's row to the next
+  const float* a2;           // [rank][H * D]: A2 transposed
+  const float* a_bias;       // [H * D]
+  int rank;
+  float q_scale, inv_tau;
+  float* state;              // [state_rows][H][D][E]
+  int state_rows;
+  const int* seq_start;
+  const int* seq_slot;
+  int H, D, E;
+};
+
+#define GLA_STEP_THREADS 512
+#define GLA_STEP_AHEAD 8     // rows of the state that a thread has under way
+
+// Single tokens: a workgroup for a (head, sequence).  The state is all that moves, once in and once out, so a wave reads it
+// in whole rows of VEC consecutive values a lane, and the first rows are asked for before the decays are made.  Thread =
+// row group * CL + column group; the row groups' sums meet in LDS, where the head's read-out is normed and gated.
+template <int VEC, typename T>
+__global__ void __launch_bounds__(GLA_STEP_THREADS)
+gla_step_kernel(GlaArgs a, const float* __restrict__ gain, float eps, const float* __restrict__ gate, T* __restrict__ out,
+                int out_ld) {
+  typedef float vec __attribute__((ext_vector_type(VEC == 1 ? 2 : VEC)));      // (one value: the first of two)
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float red[16];
+  const int D = a.D, E = a.E, tid = threadIdx.x, head = blockIdx.x, b = blockIdx.y;
+  float* qs = lds;                  // [D]
+  float* ks = qs + D;               // [D]
+  float* gs = ks + D;               // [D]
+  float* part = gs + D;             // [row groups][E]
+  const int CL = E / VEC, RG = GLA_STEP_THREADS / CL;      // (the host: E a multiple of VEC, CL at most the threads)
+  const int cl = tid % CL, rg = tid / CL;
+  const bool on = rg < RG;
+  const size_t tok = a.seq_start[b];
+  int slot = a.seq_slot[b];
+  if (slot < 0 || slot >= a.state_rows) slot = a.state_rows - 1;
+  float* S = a.state + ((size_t)slot * a.H + head) * D * E + cl * VEC;
+  auto load = [&](vec& x, int row) {
+    if (on && row < D) {
+      if constexpr (VEC == 1) x[0] = S[(size_t)row * E];
+      else x = *(const vec*)(S + (size_t)row * E);
+    }
+  };
+  vec s[GLA_STEP_AHEAD];
+#pragma unroll
+  for (int i = 0; i < GLA_STEP_AHEAD; ++i) load(s[i], rg + RG * i);
+  vec v;
+  if constexpr (VEC == 1) v[0] = on ? a.v[tok * a.ld + head * E + cl] : 0.f;
+  else
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] = on ? a.v[tok * a.ld + head * E + cl * VEC + e] : 0.f;
+  for (int d = tid; d < D; d += GLA_STEP_THREADS) {
+    const int hd = head * D + d;
+    qs[d] = a.q[tok * a.ld + hd] * a.q_scale;
+    ks[d] = a.k[tok * a.ld + hd];
+    float z = a.a_bias[hd];
+    for (int r = 0; r < a.rank; ++r) z = fmaf(a.a2[(size_t)r * a.H * D + hd], a.mid[tok * a.ld + r], z);
+    gs[d] = expf(-rc_softplus(-z) * a.inv_tau);
+  }
+  __syncthreads();
+  vec acc = {};
+  for (int row0 = rg; row0 < D; row0 += RG * GLA_STEP_AHEAD) {
+#pragma unroll
+    for (int i = 0; i < GLA_STEP_AHEAD; ++i) {
+      const int row = row0 + RG * i;
+      if (on && row < D) {
+        const float g = gs[row], kr = ks[row], qr = qs[row];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+          s[i][e] = fmaf(g, s[i][e], kr * v[e]);
+          acc[e] = fmaf(s[i][e], qr, acc[e]);
+        }
+        if constexpr (VEC == 1) S[(size_t)row * E] = s[i][0];
+        else *(vec*)(S + (size_t)row * E) = s[i];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < GLA_STEP_AHEAD; ++i) load(s[i], row0 + RG * (GLA_STEP_AHEAD + i));
+  }
+  if (on) {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) part[rg * E + cl * VEC + e] = acc[e];
+  }
+  __syncthreads();
+  float o = 0.f;
+  if (tid < E)
+    for (int r = 0; r < RG; ++r) o += part[r * E + tid];
+  const float inv = 1.f / sqrtf(block_sum(o * o, red) / (float)E + eps);
+  if (tid < E) {
+    const float g = gate[tok * a.ld + head * E + tid];
+    out[tok * out_ld + head * E + tid] = from_f32<T>(o * inv * gain[head * E + tid] * rc_silu(g));
+  }
+}
+
+// Prompts in chunks of C = 16 tokens (HDC).  With L_t = the sum of the logarithms of the decays of the chunk's tokens up to
+// t (a vector over the key channels):
+//   o_t = S^T (q_t exp(L_t)) + sum_(j<=t) A_tj v_j,   A_tj = sum_d q_td k_jd exp(L_td - L_jd)
+//   S'  = diag(exp(L_C)) S + sum_j (k_j exp(L_C - L_j)) v_j^T
+// gla_chunks_kernel makes Q exp(L), (K exp(L_C - L))^T, A and exp(L_C) for all chunks side by side; gla_carry_kernel walks a
+// head's chunks with products alone, in the layout of head_delta_carry_kernel.  None of the exponents above is positive.
+// A on the matrix cores is (Q exp(L)) (K exp(-L))^T, whose second factor grows as the chunk's decays fall: it is taken where
+// no channel loses more than exp(-GLA_SPREAD) within the chunk, and else A is summed term by term.
+#define GLA_SPREAD 60.f
+#define GLA_RANK_PIECE 64
+__host__ __device__ __forceinline__ size_t gla_chunk_floats(int NT) { return (size_t)2 * NT * 256 + 256 + 16 * NT; }
+
+__global__ void __launch_bounds__(256)
+gla_chunks_kernel(GlaArgs a, int n_seqs, float* __restrict__ work, int NT) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int LDD = 16 * NT + 1, DP = 16 * NT;
+  float* qs = lds;                          // [C][LDD] queries times q_scale, zeros beyond the keys and the chunk's tokens
+  float* ks = qs + HDC * LDD;               // [C][LDD]
+  float* Ls = ks + HDC * LDD;               // [C][LDD] L_t
+  float* mids = Ls + HDC * LDD;             // [C][GLA_RANK_PIECE]
+  float* part = mids + HDC * GLA_RANK_PIECE;      // [4 waves][C][C + 1]
+  float* red = part + 4 * HDC * (HDC + 1);        // [4]
+  int first, n;
+  if (!hd_chunk_of(blockIdx.x, a.seq_start, n_seqs, first, n)) return;      // (the whole workgroup)
+  const int head = blockIdx.y, tid = threadIdx.x, wave = tid / SYN_WAVE, lane = tid % SYN_WAVE, D = a.D;
+  for (int e = tid; e < HDC * DP; e += 256) {
+    const int t = e / DP, d = e % DP;
+    const bool in = t < n && d < D;
+    const size_t at = (size_t)(first + t) * a.ld + head * D + d;
+    qs[t * LDD + d] = in ? a.q[at] * a.q_scale : 0.f;
+    ks[t * LDD + d] = in ? a.k[at] : 0.f;
+  }
+  // the decays: a thread makes one channel's for eight tokens, then the second eight add what the first eight came to
+  for (int e0 = 0; e0 < 2 * DP; e0 += 256) {
+    const int e = e0 + tid, d = e % DP, t0 = e / DP * 8;
+    const bool mine = e < 2 * DP, in = mine && d < D;
+    float z[8];
+    const float bias = in ? a.a_bias[head * D + d] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) z[i] = bias;
+    for (int r0 = 0; r0 < a.rank; r0 += GLA_RANK_PIECE) {
+      const int nr = min(GLA_RANK_PIECE, a.rank - r0);
+      __syncthreads();
+      for (int m = tid; m < HDC * nr; m += 256)
+        mids[(m / nr) * GLA_RANK_PIECE + m % nr] = a.mid[(size_t)(first + min(m / nr, n - 1)) * a.ld + r0 + m % nr];
+      __syncthreads();
+      if (in)
+        for (int r = 0; r < nr; ++r) {
+          const float w = a.a2[(size_t)(r0 + r) * a.H * D + head * D + d];
+#pragma unroll
+          for (int i = 0; i < 8; ++i) z[i] = fmaf(w, mids[(t0 + i) * GLA_RANK_PIECE + r], z[i]);
+        }
+    }
+    float run = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      run -= (in && t0 + i < n) ? rc_softplus(-z[i]) * a.inv_tau : 0.f;      // (tokens beyond the chunk's: nothing decays)
+      z[i] = run;
+    }
+    if (mine && t0 == 0) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) Ls[i * LDD + d] = z[i];
+    }
+    __syncthreads();      // (a channel's second eight come in the turn of its first eight or in a later one)
+    if (mine && t0 != 0) {
+      const float before = Ls[7 * LDD + d];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) Ls[(8 + i) * LDD + d] = before + z[i];
+    }
+  }
+  __syncthreads();
+  float spread = 0.f;
+  for (int d = tid; d < DP; d += 256) spread = fmaxf(spread, -Ls[(HDC - 1) * LDD + d]);
+  spread = wave_max(spread);
+  if (lane == 0) red[wave] = spread;
+  __syncthreads();
+  spread = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+  const bool on_cores = spread <= GLA_SPREAD;                                  // (the same for the whole workgroup)
+  float* wf = work + ((size_t)blockIdx.x * a.H + head) * gla_chunk_floats(NT);
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  // fragments: tile of 16 channels, lane = 16 g + m; a wave's turns are tiles wave, wave + 4, ...
+  for (int e = tid; e < NT * 64; e += 256) {
+    const int tile = e / 64, m = e % 16, g = (e % 64) / 16;
+    hd_frag fq, ft;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int d = 16 * tile + 4 * g + j, dt = 16 * tile + m, t = 4 * g + j;
+      fq[j] = qs[m * LDD + d] * expf(Ls[m * LDD + d]);
+      ft[j] = ks[t * LDD + dt] * expf(Ls[(HDC - 1) * LDD + dt] - Ls[t * LDD + dt]);
+    }
+    ((hd_frag*)wf)[e] = fq, ((hd_frag*)wf)[NT * 64 + e] = ft;
+    if (on_cores) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = 16 * tile + 4 * g + j;
+        acc = hd_mfma(fq[j], ks[m * LDD + d] * expf(-Ls[m * LDD + d]), acc);
+      }
+    }
+  }
+  for (int d = tid; d < DP; d += 256) wf[2 * NT * 256 + 256 + d] = expf(Ls[(HDC - 1) * LDD + d]);
+  const int t = tid / HDC, j = tid % HDC;
+  float A = 0.f;
+  if (on_cores) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) part[(wave * HDC + 4 * (lane / 16) + i) * (HDC + 1) + lane % 16] = acc[i];
+    __syncthreads();
+#pragma unroll
+    for (int w = 0; w < 4; ++w) A += part[(w * HDC + t) * (HDC + 1) + j];
+  } else if (t >= j) {
+    for (int d = 0; d < D; ++d)
+      A = fmaf(qs[t * LDD + d] * ks[j * LDD + d], expf(Ls[t * LDD + d] - Ls[j * LDD + d]), A);
+  }
+  wf[2 * NT * 256 + ((j / 4) * 16 + t) * 4 + j % 4] = t >= j ? A : 0.f;      // row t, k = j
+}
+
+template <int TPW, int CG>
+struct GlaOperands {
+  hd_frag q[TPW], kt[TPW], A;
+  f32x4 gc[TPW], v[CG];      // exp(L_C) of the rows 4 g + j, the values of the tokens 4 g + j in this lane's columns
+};
+
+// W waves hold TPW tiles of 16 rows of a head's state each, CG groups of 16 columns a workgroup; one more wave makes and
+// stores the outputs from what the waves' rows give to Q S (through LDS, two buffers in turns: one barrier a chunk).
+template <int TPW, int W, int CG>
+__global__ void __launch_bounds__((W + 1) * SYN_WAVE)
+gla_carry_kernel(GlaArgs a, const float* __restrict__ work, float* __restrict__ o) {
+  constexpr int NT = TPW * W;
+  __shared__ __attribute__((aligned(16))) f32x4 part[2][W][CG][SYN_WAVE];
+  const int head = blockIdx.x, b = blockIdx.z, wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE;
+  const bool holds = wave < W;                       // (else the wave of the outputs)
+  const int H = a.H, D = a.D, E = a.E, g = lane / 16, col = blockIdx.y * 16 * CG + lane % 16;
+  const int s0 = a.seq_start[b], n_new = a.seq_start[b + 1] - s0;
+  if (n_new <= 0) return;                            // (the whole workgroup)
+  int slot = a.seq_slot[b];
+  if (slot < 0 || slot >= a.state_rows) slot = a.state_rows - 1;
+  float* Sg = a.state + ((size_t)slot * H + head) * D * E;
+  f32x4 S[CG][TPW];
+#pragma unroll
+  for (int y = 0; y < CG; ++y)
+#pragma unroll
+    for (int i = 0; i < TPW; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = 16 * (wave * TPW + i) + 4 * g + j, c = col + 16 * y;
+        S[y][i][j] = (holds && c < E && d < D) ? Sg[(size_t)d * E + c] : 0.f;
+      }
+  const int chunk0 = s0 / HDC + b, n_chunks = (n_new + HDC - 1) / HDC;
+  const float* vp = a.v + (size_t)s0 * a.ld + head * E;
+  float* op = o + (size_t)s0 * H * E + head * E + col;
+  auto ask = [&](GlaOperands<TPW, CG>& x, int c) {
+    c = min(c, n_chunks - 1);
+    const float* wf = work + ((size_t)(chunk0 + c) * H + head) * gla_chunk_floats(NT);
+    if (holds) {
+      const hd_frag* kf = (const hd_frag*)wf + wave * TPW * 64 + lane;
+#pragma unroll
+      for (int i = 0; i < TPW; ++i) {
+        x.q[i] = kf[i * 64], x.kt[i] = kf[(NT + i) * 64];
+        x.gc[i] = ((const f32x4*)(wf + 2 * NT * 256 + 256))[(wave * TPW + i) * 4 + g];
+      }
+    } else {
+      x.A = ((const hd_frag*)(wf + 2 * NT * 256))[lane];
+    }
+#pragma unroll
+    for (int y = 0; y < CG; ++y)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)      // (tokens beyond the last meet zeros; columns beyond are not stored)
+        x.v[y][j] = vp[(size_t)min(c * HDC + 4 * g + j, n_new - 1) * a.ld + min(col + 16 * y, E - 1)];
+  };
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  auto step = [&](const GlaOperands<TPW, CG>& x, int c, int at) {
+    if (holds) {
+#pragma unroll
+      for (int y = 0; y < CG; ++y) {
+        f32x4 qs[2] = {zero, zero};
+#pragma unroll
+        for (int i = 0; i < TPW; ++i)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) qs[j & 1] = hd_mfma(x.q[i][j], S[y][i][j], qs[j & 1]);
+        part[at][wave][y][lane] = qs[0] + qs[1];
+      }
+    }
+    __syncthreads();
+    if (holds) {
+#pragma unroll
+      for (int y = 0; y < CG; ++y) {
+#pragma unroll
+        for (int i = 0; i < TPW; ++i) S[y][i] *= x.gc[i];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int i = 0; i < TPW; ++i) S[y][i] = hd_mfma(x.kt[i][j], x.v[y][j], S[y][i]);
+      }
+    } else {
+#pragma unroll
+      for (int y = 0; y < CG; ++y) {
+        f32x4 out = part[at][0][y][lane];
+#pragma unroll
+        for (int w = 1; w < W; ++w) out += part[at][w][y][lane];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) out = hd_mfma(x.A[j], x.v[y][j], out);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int t = c * HDC + 4 * g + j;
+          if (t < n_new && col + 16 * y < E) op[(size_t)t * H * E + 16 * y] = out[j];
+        }
+      }
+    }
+  };
+  GlaOperands<TPW, CG> even, odd;
+  ask(even, 0), ask(odd, 1);
+  for (int c = 0; c < n_chunks; c += 2) {
+    step(even, c, 0);
+    ask(even, c + 2);
+    if (c + 1 < n_chunks) {
+      step(odd, c + 1, 1);
+      ask(odd, c + 3);
+    }
+  }
+#pragma unroll
+  for (int y = 0; y < CG; ++y)
+#pragma unroll
+    for (int i = 0; i < TPW; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = 16 * (wave * TPW + i) + 4 * g + j, c = col + 16 * y;
+        if (holds && c < E && d < D) Sg[(size_t)d * E + c] = S[y][i][j];
+      }
+}
+
+static int gla_check(const char* name, const GlaArgs& a, int n_seqs) {
+  SYN_CHECK(n_seqs > 0 && a.H > 0 && a.D > 0 && a.E > 0 && a.rank > 0, "%s: empty input", name);
+  SYN_CHECK(a.D <= RC_ROWS_MAX, "%s: keys of %d values (at most %d)", name, a.D, RC_ROWS_MAX);
+  SYN_CHECK(a.ld >= a.H * max(a.D, a.E) && a.ld >= a.rank && a.state_rows > 0, "%s: rows of %d values", name, a.ld);
+  return 0;
+}
+
+// floats of scratch memory of gated_linear_scan
+SYN_EXPORT long syn_gated_linear_scratch(int n_tokens, int n_seqs, int H, int D) {
+  return ((long)n_tokens / HDC + n_seqs) * H * (long)gla_chunk_floats(hd_tiles(D));
+}
+
+// any number of new tokens a sequence; o [n_tokens][H * E] float
+SYN_EXPORT int syn_gated_linear_scan(const float* q, const float* k, const float* v, const float* mid, int ld, const float* a2,
+                                     const float* a_bias, int rank, float q_scale, float inv_tau, float* state, int state_rows,
+                                     const int* seq_start, const int* seq_slot, int n_seqs, int n_tokens, int H, int D, int E,
+                                     float* o, float* scratch, hipStream_t stream) {
+  const GlaArgs a = {q, k, v, mid, ld, a2, a_bias, rank, q_scale, inv_tau, state, state_rows, seq_start, seq_slot, H, D, E};
+  if (int rc = gla_check("gated_linear_scan", a, n_seqs)) return rc;
+  SYN_CHECK(n_tokens > 0 && scratch && (uintptr_t)scratch % 16 == 0, "gated_linear_scan: the scratch memory is not aligned");
+  const int NT = hd_tiles(D), chunks = n_tokens / HDC + n_seqs;
+  const size_t bytes = (3 * HDC * (16 * NT + 1) + HDC * GLA_RANK_PIECE + 4 * HDC * (HDC + 1) + 4) * sizeof(float);
+  gla_chunks_kernel<<<dim3(chunks, H), 256, bytes, stream>>>(a, n_seqs, scratch, NT);
+  SYN_LAUNCH_CHECK("gla_chunks");
+  const int groups = (E + 15) / 16;
+  const bool wide = (long)H * n_seqs * ((groups + 1) / 2) >= 2L * syn_compute_units();
+  const dim3 grid(H, wide ? (groups + 1) / 2 : groups, n_seqs);
+#define SYN_GLA2(T, W, CG) gla_carry_kernel<T, W, CG><<<grid, (W + 1) * SYN_WAVE, 0, stream>>>(a, scratch, o)
+#define SYN_GLA(T, W)                 \
+  case T * W:                         \
+    if (wide) SYN_GLA2(T, W, 2);      \
+    else SYN_GLA2(T, W, 1);           \
+    break
+  switch (NT) {
+    SYN_GLA(1, 1); SYN_GLA(1, 2); SYN_GLA(1, 4); SYN_GLA(2, 4); SYN_GLA(3, 4); SYN_GLA(4, 4);
+    default: SYN_CHECK(false, "gated_linear_scan: keys of %d values", D);
+  }
+#undef SYN_GLA2
+#undef SYN_GLA
+  SYN_LAUNCH_CHECK("gla_carry");
+  return 0;
+}
+
+// one new token a sequence; out [n_seqs] rows of out_ld values: each head's read-out over its root mean square, times gain
+// [H * E], times silu(gate) (columns of the projection's rows)
+SYN_EXPORT int syn_gated_linear_step(const float* q, const float* k, const float* v, const float* mid, int ld, const float* a2,
+                                     const float* a_bias, int rank, float q_scale, float inv_tau, float* state, int state_rows,
+                                     const int* seq_start, const int* seq_slot, int n_seqs, int H, int D, int E,
+                                     const float* gain, float eps, const float* gate, void* out, int out_ld, int out_is_f32,
+                                     hipStream_t stream) {
+  const GlaArgs a = {q, k, v, mid, ld, a2, a_bias, rank, q_scale, inv_tau, state, state_rows, seq_start, seq_slot, H, D, E};
+  if (int rc = gla_check("gated_linear_step", a, n_seqs)) return rc;
+  SYN_CHECK(E <= GLA_STEP_THREADS, "gated_linear_step: values of %d (at most %d)", E, GLA_STEP_THREADS);
+  SYN_CHECK(gain && gate && out && out_ld >= H * E, "gated_linear_step: result rows of %d values", out_ld);
+  const bool four = E % 4 == 0 && (uintptr_t)state % 16 == 0;
+  const int row_groups = GLA_STEP_THREADS / (four ? E / 4 : E);
+  const size_t bytes = (3 * (size_t)D + (size_t)row_groups * E) * sizeof(float);
+  const dim3 grid(H, n_seqs);
+#define SYN_GLAS(VEC, T) gla_step_kernel<VEC, T><<<grid, GLA_STEP_THREADS, bytes, stream>>>(a, gain, eps, gate, (T*)out, out_ld)
+  if (out_is_f32) {
+    if (four) SYN_GLAS(4, float); else SYN_GLAS(1, float);
+  } else {
+    if (four) SYN_GLAS(4, bf16); else SYN_GLAS(1, bf16);
+  }
+#undef SYN_GLAS
+  SYN_LAUNCH_CHECK("gated_linear_step");
   return 0;
 }
 

@@ -165,9 +165,11 @@ def _activation_args(activation):
 
 # ----------------------------------------------------------------------------- rows
 
-def embed(table, ids, resid, scale=1.0):
+def embed(table, ids, resid, scale=1.0, sinusoid=None, keep=None):
     """resid[n, :] = scale * table[ids[n], :] as float.  table [V, H] bf16|f32 (or bf16 in fragment order, pack_weight: four
-    dimensions), ids [N] int32, resid [N, H] f32."""
+    dimensions), ids [N] int32, resid [N, H] f32.
+    sinusoid = (rates float64 [(H + 1) / 2], positions int32 [N]): sin(p f_i) is added at column 2 i and cos(p f_i) at
+    2 i + 1 for the row's position p.  keep [N, H] f32: receives the same rows as resid."""
     if isinstance(table, torch.Tensor) and table.dim() == 4:
         _need(table, "embed.table", _BF16, (None, None, 64, 8))
         H, kind = table.shape[1] * 32, 2
@@ -176,8 +178,24 @@ def embed(table, ids, resid, scale=1.0):
         H, kind = table.shape[1], _is_f32(table)
     _need(ids, "embed.ids", _I32, (None,))
     _need(resid, "embed.resid", _F32, (ids.shape[0], H))
+    rates = pos = None
+    if sinusoid is not None:
+        rates, pos = sinusoid
+        _need(rates, "embed.rates", torch.float64, ((H + 1) // 2,))
+        _need(pos, "embed.positions", _I32, (ids.shape[0],))
+    if keep is not None:
+        _need(keep, "embed.keep", _F32, (ids.shape[0], H))
     _call(load_library("core"), "syn_embed", _ptr(table), kind, _ptr(ids), _ptr(resid), ids.shape[0], H,
-          ctypes.c_float(scale), _stream())
+          ctypes.c_float(scale), _ptr(rates), _ptr(pos), _ptr(keep), _stream())
+
+
+def soft_cap(x, cap):
+    """x <- cap * tanh(x / cap), float, in place."""
+    _need(x, "soft_cap.x", _F32)
+    if not cap > 0.0:
+        raise KernelError(f"soft_cap: a cap of {cap}")
+    if x.numel():
+        _call(load_library("core"), "syn_soft_cap", _ptr(x), ctypes.c_long(x.numel()), ctypes.c_float(cap), _stream())
 
 
 def add_rmsnorm(resid, delta, gain, eps, out, rows=None, gain_offset=0.0):
@@ -240,12 +258,15 @@ def _packed_shape(w, name, K):
 # What the sums of a plain product may pass before they are stored (point_activation in csrc/common.h): the activation of an
 # ungated feed-forward.  "relu_squared": max(z, 0)^2
 POINT_ACTIVATIONS = {"relu_squared": 1}
+POINT_SOFTCAP = 2        # the pair ("softcap", cap): cap * tanh(z / cap), in the products for few rows only
 
 
 def point_code(name) -> int:
     if name is None:
         return 0
-    if name not in POINT_ACTIVATIONS:
+    if isinstance(name, (tuple, list)) and len(name) == 2 and name[0] == "softcap" and float(name[1]) > 0.0:
+        return POINT_SOFTCAP
+    if not isinstance(name, str) or name not in POINT_ACTIVATIONS:
         raise KernelError(f"activation {name!r}: the plain products apply {sorted(POINT_ACTIVATIONS)}")
     return POINT_ACTIVATIONS[name]
 
@@ -273,9 +294,13 @@ def gemm(x, w, out, force_simt=False, point=None):
             for m0 in range(0, M, PACKED_BLOCK_ROWS):
                 gemm_packed(x[m0:m0 + PACKED_BLOCK_ROWS], w, rows[m0:m0 + PACKED_BLOCK_ROWS], point=point)
             return
+        if point_of == POINT_SOFTCAP:
+            raise KernelError("gemm: the tiles have no soft cap (ops.soft_cap behind the product)")
     else:
         _need(w, "gemm.w", x.dtype, (None, K))
         N = w.shape[0]
+        if point_of == POINT_SOFTCAP:
+            raise KernelError("gemm: the tiles have no soft cap (ops.soft_cap behind the product)")
     slices = 1
     if out.dim() == 3:
         slices = out.shape[0]
@@ -367,7 +392,8 @@ def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, res
     the sums are added into resid, xs = (gain_offset + gain) * resid, ss = sums of resid^2 over groups of 16 columns;
     row_scale = (ss [M, G] float, dim, eps): the sums of row m are multiplied by rsqrt(sum(ss[m]) / dim + eps), which
     makes this the product over the normed rows when x is the xs that came with ss.
-    point: as for gemm (behind the row's factor)."""
+    resid_norm may go on with (add_rows [M, N] float or None, add_vec [N] float or None): what else is added into resid.
+    point: as for gemm (behind the row's factor), or ("softcap", cap)."""
     point_of = point_code(point)
     _need(x, "gemm_packed.x", _BF16, (None, None))
     M, K = x.shape
@@ -378,7 +404,7 @@ def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, res
     if M > 16 or (paired and N % 32):
         raise KernelError(f"gemm_packed: M = {M} (at most 16), N = {N}")
     slices = 1
-    ss = resid = xs = ss_out = gain = None
+    ss = resid = xs = ss_out = gain = add_rows = add_vec = None
     groups = dim = 0
     eps = gain_offset = 0.0
     if row_scale is not None:
@@ -388,7 +414,12 @@ def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, res
         if groups < 1 or dim < 1:
             raise KernelError(f"gemm_packed: a row statistic of {groups} groups over {dim} columns")
     if resid_norm is not None:
-        resid, gain, gain_offset, xs, ss_out = resid_norm
+        resid, gain, gain_offset, xs, ss_out = resid_norm[:5]
+        add_rows, add_vec = resid_norm[5:] if len(resid_norm) > 5 else (None, None)
+        if add_rows is not None:
+            _need(add_rows, "gemm_packed.add_rows", _F32, (M, N))
+        if add_vec is not None:
+            _need(add_vec, "gemm_packed.add_vec", _F32, (N,))
         if paired or out is not None:
             raise KernelError("gemm_packed: the product before a norm is not gated and has no output beside resid, xs and ss")
         _need(resid, "gemm_packed.resid", _F32, (M, N))
@@ -406,14 +437,17 @@ def gemm_packed(x, wp, out, paired=False, activation="silu", row_scale=None, res
     else:
         _need(out, "gemm_packed.out", (_BF16, _F32), (M, N))
         out_code = 2 if out.dtype == _F32 else 1
+    act = _activation_args(activation)
+    if point_of == POINT_SOFTCAP:        # (a plain product applies no gated activation: the bound is the cap)
+        act = (act[0], ctypes.c_float(float(point[1])))
     if row_scale is None and resid_norm is None:
         _call(load_library("core"), "syn_gemm_packed", _ptr(x), _ptr(wp), _ptr(out), out_code,
-              M, N, K, 1 if paired else 0, *_activation_args(activation), slices, point_of, _stream())
+              M, N, K, 1 if paired else 0, *act, slices, point_of, _stream())
         return
     _call(load_library("core"), "syn_gemm_packed_norm", _ptr(x), _ptr(wp), _ptr(out), out_code, M, N, K,
-          1 if paired else 0, *_activation_args(activation), slices, _ptr(ss), int(groups), int(dim), ctypes.c_float(eps),
+          1 if paired else 0, *act, slices, _ptr(ss), int(groups), int(dim), ctypes.c_float(eps),
           _ptr(resid), _ptr(xs), _ptr(ss_out), _ptr(gain), _is_f32(gain) if gain is not None else 0,
-          ctypes.c_float(gain_offset), point_of, _stream())
+          ctypes.c_float(gain_offset), _ptr(add_rows), _ptr(add_vec), point_of, _stream())
 
 
 _compute_units = None
@@ -846,7 +880,7 @@ def _check_window_pages(k_pages, v_pages, dtype, nkv, dim, vdim, name, v_share=1
 def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_pos, q_gain, k_gain, eps,
                   n_heads, n_kv_heads, dim, vdim, write_kv=True, rotation=None, v_share=1, pairs=False,
                   norm_whole=False, values_are_keys=False, q_temp=None):
-    """proj [N, width] float: the fused projection [q | k | v | ...]; bias float [>= q, k, v columns] or None.  q and k
+    """proj [N, width] float (or such columns of longer rows): the fused projection [q | k | v | ...]; bias float [>= q, k, v columns] or None.  q and k
     heads get their bias and (with gains, float [dim]) an RMSNorm over the head; q goes to q_out [N, nh * dim], k and v
     (with its bias) into the pages of sequence tok_seq[n] at position tok_pos[n].
     rotation = (cos, sin) float [positions, rot / 2]: the first `rot` values of every q and k head are then turned by
@@ -858,8 +892,8 @@ def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_
     are the keys as projected (with their bias, before norm and rotation).  q_temp = (coef, every): queries at position p
     are multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
     nh, nkv = n_heads, n_kv_heads
-    _need(proj, "window_intake.proj", _F32, (None, None))
-    N, width = proj.shape
+    N = tok_pos.shape[0]
+    width = _float_rows_view(proj, "window_intake.proj", N, 1)
     if v_share < 1 or nkv % v_share:
         raise KernelError(f"window_intake: {nkv} kv heads in shares of {v_share} value heads")
     nv = nkv // v_share
@@ -889,6 +923,8 @@ def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_
             raise KernelError(f"window_intake: a rotation of {rot} values of heads of {dim}")
     _need(tok_seq, "window_intake.tok_seq", _I32, (N,))
     _need(tok_pos, "window_intake.tok_pos", _I32, (N,))
+    if proj.shape[1] < used:
+        raise KernelError(f"window_intake: rows of {proj.shape[1]} values do not hold {'q, k and v' if write_kv else 'q'} ({used})")
     if (q_gain is None) != (k_gain is None):
         raise KernelError("window_intake: q and k gains come together")
     if q_gain is not None:
@@ -905,7 +941,7 @@ def window_intake(proj, bias, q_out, k_pages, v_pages, page_table, tok_seq, tok_
 
 def window_attention(q, k_pages, v_pages, page_table, tok_seq, tok_pos, out, scale, n_heads, n_kv_heads, dim, vdim,
                      window=0, keep_first=0, sink_one=False, slopes=None, log_bias=None, softcap=0.0, gate=None,
-                     gate_bias=None, v_share=1, sinks=None, chunk=0, gate_per_head=False):
+                     gate_bias=None, v_share=1, sinks=None, chunk=0, gate_per_head=False, out_scale=1.0):
     """v_share: that many neighbouring kv heads read the values of one value head (v_pages holds nkv / v_share heads).
     Attention of every token (prompts and single tokens alike) whose query is q [N, nh * dim] over the pages
     (which already hold the tokens): score = scale q.k [soft cap] - slopes[h] (i - j) - r1[h] ln(1 + r2[h] (i - j))
@@ -913,7 +949,8 @@ def window_attention(q, k_pages, v_pages, page_table, tok_seq, tok_pos, out, sca
     j < keep_first) and (no chunk or j // chunk == i // chunk or j < keep_first); sink_one: one more in the softmax's
     denominator; sinks float [nh]: exp(sinks[h]) more (a learned score of a key without a value); gate: a float view
     [N, >= nh * vdim] (with gate_per_head [N, >= nh]: one number a head) with row stride gate.stride(0) whose sigmoid
-    multiplies the result; out [N, nh * vdim] in q's type."""
+    multiplies the result; out_scale: a factor on the result; out [N, nh * vdim] in q's type (columns of longer rows, if
+    its rows are)."""
     nh, nkv = n_heads, n_kv_heads
     _need(q, "window_attention.q", (_BF16, _F32), (None, nh * dim))
     N = q.shape[0]
@@ -921,7 +958,7 @@ def window_attention(q, k_pages, v_pages, page_table, tok_seq, tok_pos, out, sca
     _need(page_table, "window_attention.page_table", _I32, (None, None))
     _need(tok_seq, "window_attention.tok_seq", _I32, (N,))
     _need(tok_pos, "window_attention.tok_pos", _I32, (N,))
-    _need(out, "window_attention.out", q.dtype, (N, nh * vdim))
+    ldo = _rows_view(out, "window_attention.out", q.dtype, N, nh * vdim)
     if max(dim, vdim) > WINDOW_ATTENTION_MAX_DIM:
         raise KernelError(f"window_attention: head sizes {dim}, {vdim} exceed {WINDOW_ATTENTION_MAX_DIM}")
     r1 = r2 = None
@@ -942,7 +979,8 @@ def window_attention(q, k_pages, v_pages, page_table, tok_seq, tok_pos, out, sca
           _ptr(page_table), page_table.shape[1], _ptr(tok_seq), _ptr(tok_pos), _ptr(gate), gate_stride,
           _ptr(gate_bias if gate is not None else None), _ptr(out), ctypes.c_float(scale), N, nh, nkv, dim, vdim,
           _ptr(slopes), _ptr(r1), _ptr(r2), ctypes.c_float(float(softcap or 0.0)), int(window or 0), int(keep_first or 0),
-          1 if sink_one else 0, int(v_share), _ptr(sinks), int(chunk or 0), 1 if gate_per_head else 0, _stream())
+          1 if sink_one else 0, int(v_share), _ptr(sinks), int(chunk or 0), 1 if gate_per_head else 0, ldo,
+          ctypes.c_float(out_scale), _stream())
 
 
 def _sink_and_chunk(name, sinks, sink_one, chunk, n_heads):
@@ -965,7 +1003,7 @@ def window_prefill_takes(dim, vdim) -> bool:
 def window_attention_prefill_bf16(q, k_pages, v_pages, page_table, seq_start, seq_past, out, scale, n_heads, n_kv_heads,
                                   dim, vdim, window=0, keep_first=0, sink_one=False, slopes=None, log_bias=None,
                                   softcap=0.0, gate=None, gate_bias=None, v_share=1, sinks=None, chunk=0,
-                                  gate_per_head=False):
+                                  gate_per_head=False, out_scale=1.0):
     """window_attention for the new tokens of each sequence of a step in bf16, on the matrix cores: seq_start [B + 1]
     offsets of the sequences' new tokens in q, seq_past [B] tokens cached before (the pages already hold the new
     ones).  Scores and weights are 32-bit; a weight meets V as two bf16 numbers (16 bits of mantissa)."""
@@ -981,7 +1019,7 @@ def window_attention_prefill_bf16(q, k_pages, v_pages, page_table, seq_start, se
     _need(seq_past, "window_attention_prefill.seq_past", _I32, (B,))
     if page_table.shape[0] < B:
         raise KernelError(f"window_attention_prefill: page table has {page_table.shape[0]} rows for {B} sequences")
-    _need(out, "window_attention_prefill.out", _BF16, (N, nh * vdim))
+    ldo = _rows_view(out, "window_attention_prefill.out", _BF16, N, nh * vdim)
     r1 = r2 = None
     if log_bias is not None:
         r1, r2 = log_bias
@@ -1000,7 +1038,18 @@ def window_attention_prefill_bf16(q, k_pages, v_pages, page_table, seq_start, se
           _ptr(page_table), page_table.shape[1], _ptr(seq_start), _ptr(seq_past), B, N, _ptr(gate), gate_stride,
           _ptr(gate_bias if gate is not None else None), _ptr(out), ctypes.c_float(scale), nh, nkv, dim, vdim,
           _ptr(slopes), _ptr(r1), _ptr(r2), ctypes.c_float(float(softcap or 0.0)), int(window or 0), int(keep_first or 0),
-          1 if sink_one else 0, int(v_share), _ptr(sinks), int(chunk or 0), 1 if gate_per_head else 0, _stream())
+          1 if sink_one else 0, int(v_share), _ptr(sinks), int(chunk or 0), 1 if gate_per_head else 0, ldo,
+          ctypes.c_float(out_scale), _stream())
+
+
+def _rows_view(t, name, dtypes, n_rows, n_cols):
+    """A result [n_rows, n_cols] whose rows may be pieces of longer rows: returns the row stride in elements."""
+    dtypes = dtypes if isinstance(dtypes, (tuple, list)) else (dtypes,)
+    if not isinstance(t, torch.Tensor) or t.dtype not in dtypes or not t.is_cuda or tuple(t.shape) != (n_rows, n_cols):
+        raise KernelError(f"{name}: expected [{n_rows}, {n_cols}] {' or '.join(str(d) for d in dtypes)} on the GPU")
+    if (t.stride(1) != 1 and n_cols > 1) or (t.stride(0) < n_cols and n_rows > 1):
+        raise KernelError(f"{name}: strides {list(t.stride())} for rows of {n_cols}")
+    return max(t.stride(0), n_cols)
 
 
 def _float_rows_view(t, name, n_rows, n_cols):
@@ -1062,7 +1111,8 @@ def matrix_memory_scan(proj, i_bias, f_bias, gate_cap, q_scale, state, seq_start
 
 def head_norm_gate(o, gain, eps, gate, out, n_heads, vdim, silu_first=False, silu=False):
     """out[n, h] = o[n, h] / rms(o[n, h]) * gain[h] * sigmoid(gate[n, h]): o [N, H * vdim] float, gain float [H * vdim]
-    or None, gate a float view [N, >= H * vdim] (see _float_rows_view) or None, out [N, H * vdim] bf16 or float.
+    or None, gate a float view [N, >= H * vdim] (see _float_rows_view) or None, out [N, H * vdim] bf16 or float (or such
+    columns of longer rows).
     silu_first: the gate comes before the norm, x = o * silu(gate), out = x / rms(x) * gain; silu: behind it, but as
     silu(gate) instead of sigmoid(gate)."""
     if silu_first and silu:
@@ -1072,9 +1122,9 @@ def head_norm_gate(o, gain, eps, gate, out, n_heads, vdim, silu_first=False, sil
     if gain is not None:
         _need(gain, "head_norm_gate.gain", _F32, (n_heads * vdim,))
     stride = _float_rows_view(gate, "head_norm_gate.gate", N, n_heads * vdim) if gate is not None else 0
-    _need(out, "head_norm_gate.out", (_BF16, _F32), (N, n_heads * vdim))
+    out_stride = _rows_view(out, "head_norm_gate.out", (_BF16, _F32), N, n_heads * vdim)
     _call(load_library("core"), "syn_head_norm_gate", _ptr(o), _ptr(gain), ctypes.c_float(eps), _ptr(gate), stride,
-          _ptr(out), _is_f32(out), N, n_heads, vdim, 1 if silu_first else (2 if silu else 0), _stream())
+          _ptr(out), out_stride, _is_f32(out), N, n_heads, vdim, 1 if silu_first else (2 if silu else 0), _stream())
 
 
 # ----------------------------------------------------------------------------- short convolutions and scans over a state
@@ -1198,6 +1248,68 @@ def head_delta_scan(qkv, beta, a, a_bias, a_log, q_scale, unit_eps, state, seq_s
                 n_key_heads, dim, vdim, n_heads, not chunked, (qkv.shape[0], _ptr(work)))
 
 
+GATED_LINEAR_MAX_VDIM = 512
+
+
+def _gated_linear(name, q, k, v, mid, a2, a_bias, state, n_heads, dim, vdim, N):
+    """The checks that both forms share: the rows' common stride."""
+    H = n_heads
+    if dim > SCAN_MAX_ROWS:
+        raise KernelError(f"{name}: keys of {dim} values (at most {SCAN_MAX_ROWS})")
+    _need(a2, name + ".a2", _F32, (None, H * dim))
+    rank = a2.shape[0]
+    ld = {_float_rows_view(t, f"{name}.{n}", N, c) for t, n, c in
+          ((q, "q", H * dim), (k, "k", H * dim), (v, "v", H * vdim), (mid, "mid", rank))}
+    if len(ld) != 1:
+        raise KernelError(f"{name}: q, k, v and mid are columns of the same rows")
+    _need(a_bias, name + ".a_bias", _F32, (H * dim,))
+    _need(state, name + ".state", _F32, (None, H, dim, vdim))
+    return ld.pop(), rank
+
+
+def gated_linear_scan(q, k, v, mid, a2, a_bias, q_scale, tau, state, seq_start, seq_slot, out, n_heads, dim, vdim, scratch=None):
+    """Gated linear attention over the new tokens of every sequence of the step, in order, 16 at a time on the matrix cores
+    in 32-bit:   g = sigmoid(mid . a2 + a_bias)^(1 / tau)  for each (head, key channel);
+    S <- diag(g) S + k v^T,  o = S^T (q_scale q).
+    q, k float views [N, H * dim], v [N, H * vdim], mid [N, rank]: columns of one projection's rows; a2 float
+    [rank, H * dim] (the decays' second matrix, transposed), a_bias float [H * dim]; state float [rows, H, dim, vdim] (row
+    seq_slot[b]; a negative slot: the last row); out float [N, H * vdim].  scratch: a function (name, floats) -> float tensor
+    for the chunks' operands (StepContext.scratch; default: a new tensor)."""
+    _need(out, "gated_linear_scan.out", _F32, (None, n_heads * vdim))
+    N = out.shape[0]
+    ld, rank = _gated_linear("gated_linear_scan", q, k, v, mid, a2, a_bias, state, n_heads, dim, vdim, N)
+    B = _step_seqs("gated_linear_scan", seq_start, seq_slot)
+    lib = load_library("core")
+    lib.syn_gated_linear_scratch.restype = ctypes.c_long
+    need = lib.syn_gated_linear_scratch(N, B, n_heads, dim)
+    work = scratch("gated_linear_chunks", need) if scratch is not None else torch.empty(need, dtype=_F32, device=out.device)
+    _need(work, "gated_linear_scan.scratch", _F32)
+    if work.numel() < need:
+        raise KernelError(f"gated_linear_scan: scratch of {work.numel()} floats, {need} are needed")
+    _call(lib, "syn_gated_linear_scan", _ptr(q), _ptr(k), _ptr(v), _ptr(mid), ld, _ptr(a2), _ptr(a_bias), rank,
+          ctypes.c_float(q_scale), ctypes.c_float(1.0 / tau), _ptr(state), state.shape[0], _ptr(seq_start), _ptr(seq_slot), B, N,
+          n_heads, dim, vdim, _ptr(out), _ptr(work), _stream())
+
+
+def gated_linear_step(q, k, v, mid, a2, a_bias, q_scale, tau, state, seq_start, seq_slot, gain, eps, gate, out, n_heads, dim,
+                      vdim):
+    """gated_linear_scan for steps that bring one token a sequence, and what follows it (head_norm_gate with silu):
+    out[n, h] = o[n, h] / rms(o[n, h]) * gain[h] * silu(gate[n, h]).  gain float [H * vdim], gate a float view
+    [N, H * vdim] of the same rows, out [N, H * vdim] bf16 or float (or such columns of longer rows)."""
+    N = seq_slot.shape[0]
+    out_ld = _rows_view(out, "gated_linear_step.out", (_BF16, _F32), N, n_heads * vdim)
+    ld, rank = _gated_linear("gated_linear_step", q, k, v, mid, a2, a_bias, state, n_heads, dim, vdim, N)
+    if _float_rows_view(gate, "gated_linear_step.gate", N, n_heads * vdim) != ld:
+        raise KernelError("gated_linear_step: the gate is columns of the same rows")
+    if vdim > GATED_LINEAR_MAX_VDIM:
+        raise KernelError(f"gated_linear_step: values of {vdim} (at most {GATED_LINEAR_MAX_VDIM})")
+    _need(gain, "gated_linear_step.gain", _F32, (n_heads * vdim,))
+    B = _step_seqs("gated_linear_step", seq_start, seq_slot)
+    _call(load_library("core"), "syn_gated_linear_step", _ptr(q), _ptr(k), _ptr(v), _ptr(mid), ld, _ptr(a2), _ptr(a_bias), rank,
+          ctypes.c_float(q_scale), ctypes.c_float(1.0 / tau), _ptr(state), state.shape[0], _ptr(seq_start), _ptr(seq_slot), B,
+          n_heads, dim, vdim, _ptr(gain), ctypes.c_float(eps), _ptr(gate), _ptr(out), out_ld, _is_f32(out), _stream())
+
+
 def diff_heads(a, out, lam, eps, post, n_kv_heads, heads_per_kv, vdim):
     """Two softmax maps over the same values joined: a [N, G * 2 * R * vdim] holds, for each of the G kv heads, the R
     heads' results of the first map and then of the second; out [N, G * R * vdim] = rms_norm(a1 - lam a2) * post for
@@ -1286,15 +1398,19 @@ def measure_ceilings(device="cuda:0", read_bytes=1 << 30, repeats=5):
 
 # ----------------------------------------------------------------------------- scaled residual terms
 
-def add_scaled_rmsnorm(resid, terms, gain, eps, out, rows=None):
-    """resid += sum_t scale_t * delta_t for up to two terms (delta float [N, H] or partial sums [S, N, H], scale float
+def add_scaled_rmsnorm(resid, terms, gain, eps, out, rows=None, add_rows=None, add_vec=None):
+    """resid += sum_t scale_t * delta_t [+ add_rows [N, H] float] [+ add_vec [H] float] for up to two terms (delta float [N, H] or partial sums [S, N, H], scale float
     [H] or None), then out = RMSNorm(resid) * gain when `out` is given.  rows [n] int32: only those rows are summed and
     normed, resid is not written.  A term may be a triple (delta, scale, row_gate): row_gate a float view [N, 1] (a
     column of longer rows) whose sigmoid multiplies the term's rows."""
     _need(resid, "add_scaled_rmsnorm.resid", _F32, (None, None))
     N, H = resid.shape
-    if not 1 <= len(terms) <= 2:
+    if len(terms) > 2 or (not terms and add_rows is None and add_vec is None):
         raise KernelError(f"add_scaled_rmsnorm: {len(terms)} terms (one or two)")
+    if add_rows is not None:
+        _need(add_rows, "add_scaled_rmsnorm.add_rows", _F32, (N, H))
+    if add_vec is not None:
+        _need(add_vec, "add_scaled_rmsnorm.add_vec", _F32, (H,))
     args, gates = [], []
     for i, term in enumerate(terms):
         d, s = term[0], term[1]
@@ -1305,7 +1421,7 @@ def add_scaled_rmsnorm(resid, terms, gain, eps, out, rows=None):
             _need(s, f"add_scaled_rmsnorm.scale{i}", _F32, (H,))
         args += [_ptr(d), parts, _ptr(s)]
         gates += [_ptr(g), 0 if g is None else _float_rows_view(g, f"add_scaled_rmsnorm.row_gate{i}", N, 1)]
-    if len(terms) == 1:
+    for _ in range(2 - len(terms)):
         args += [_ptr(None), 1, _ptr(None)]
         gates += [_ptr(None), 0]
     n_out = N
@@ -1317,7 +1433,8 @@ def add_scaled_rmsnorm(resid, terms, gain, eps, out, rows=None):
         _need(out, "add_scaled_rmsnorm.out", (_BF16, _F32), (n_out, H))
     elif rows is not None:
         raise KernelError("add_scaled_rmsnorm: gathered rows without an output")
-    _call(load_library("core"), "syn_add_scaled_rmsnorm", _ptr(resid), N, _ptr(rows), n_out, *args, *gates, _ptr(gain),
+    _call(load_library("core"), "syn_add_scaled_rmsnorm", _ptr(resid), N, _ptr(rows), n_out, *args, *gates, _ptr(add_rows),
+          _ptr(add_vec), _ptr(gain),
           0 if gain is None else _is_f32(gain), ctypes.c_float(eps), _ptr(out), 0 if out is None else _is_f32(out), H,
           _stream())
 
@@ -1395,11 +1512,12 @@ def route_sort(ids, weights, n_experts):
     return seg, lists[0], lists[1], lists[2], weight_of
 
 
-def route_scores(logits, correction, ids, weights, n_groups=1, keep_groups=1, renorm=False, scale=1.0):
-    """A router that scores every expert: s = softmax(logits [N, E] float) over all E; the choice is made on
+def route_scores(logits, correction, ids, weights, n_groups=1, keep_groups=1, renorm=False, scale=1.0, sigmoid=False,
+                 group_two=False, renorm_eps=0.0):
+    """A router that scores every expert: s = softmax(logits [N, E] float) over all E (sigmoid: the sigmoid of each); the choice is made on
     s + correction [E] among the members of the keep_groups best of n_groups equal groups of neighbours (a group's
-    score: its largest choice score); ids [N, top] int32 the chosen (largest first, the lower index of equal ones),
-    weights [N, top] float their s, divided by their sum with renorm, times `scale`.  logits may be the first columns of
+    score: its largest choice score; group_two: the sum of its two largest); ids [N, top] int32 the chosen (largest first, the lower index of equal ones),
+    weights [N, top] float their s, divided by their sum (+ renorm_eps) with renorm, times `scale`.  logits may be the first columns of
     longer rows (a view with a row stride)."""
     if isinstance(logits, torch.Tensor) and logits.dim() == 2:
         ld = _float_rows_view(logits, "route_scores.logits", logits.shape[0], logits.shape[1])
@@ -1416,7 +1534,8 @@ def route_scores(logits, correction, ids, weights, n_groups=1, keep_groups=1, re
     if not 0 < top <= min(keep_groups * (E // n_groups), ROUTE_MAX_TOP):
         raise KernelError(f"route_scores: the {top} largest of {keep_groups} groups of {E // n_groups} (at most {ROUTE_MAX_TOP})")
     _call(load_library("core"), "syn_route_scores", _ptr(logits), _ptr(correction), _ptr(ids), _ptr(weights), N, E, ld, top,
-          int(n_groups), int(keep_groups), 1 if renorm else 0, ctypes.c_float(float(scale)), _stream())
+          int(n_groups), int(keep_groups), 1 if renorm else 0, ctypes.c_float(float(scale)), 1 if sigmoid else 0,
+          1 if group_two else 0, ctypes.c_float(float(renorm_eps)), _stream())
 
 
 def route_identity(x, out, seg, first, last, a_rows, o_rows, weight_of):
@@ -1452,12 +1571,15 @@ def pair_expert_rows(gate, up):
     return torch.stack([gate, up], 2).reshape(E, 2 * J, K).contiguous()
 
 
-def experts_product(x, w, out, seg, a_rows, o_rows, row_weight=None, gelu=False, force_simt=False, gated=None):
+EXPERT_ACTIVATIONS = {None: 0, "gelu": 1, "relu_squared": 2}      # the exact (erf) form; max(z, 0)^2
+
+
+def experts_product(x, w, out, seg, a_rows, o_rows, row_weight=None, act=None, force_simt=False, gated=None):
     """out[o_rows[r]] = epilogue(x[a_rows[r]] . w[e]^T) for the places r of each expert e's segment.  x [*, K] in the
     engine's type, w [E, J, K] in that type (or bf16 in fragment order, pack_expert_weights: five dimensions), out
     [*, J] in that type or float; the index lists come from route_sort and
-    must stay inside x and out (the caller sees to that: they are on the device).  Epilogue: the exact GELU, then the
-    row's weight, each if asked for.  gated: an activation of the gated products (ACTIVATIONS; one with a bound as the
+    must stay inside x and out (the caller sees to that: they are on the device).  Epilogue: an activation `act` of
+    EXPERT_ACTIVATIONS, then the row's weight, each if asked for.  gated: an activation of the gated products (ACTIVATIONS; one with a bound as the
     pair (name, bound)): w then holds gate and up rows in turns (pair_expert_rows), and out [*, J / 2] receives the
     activation of each pair of sums.  force_simt: as in heads_product."""
     _need(x, "experts_product.x", (_BF16, _F32), (None, None))
@@ -1471,8 +1593,10 @@ def experts_product(x, w, out, seg, a_rows, o_rows, row_weight=None, gelu=False,
         _need(w, "experts_product.w", x.dtype, (None, None, K))
         E, J = w.shape[0], w.shape[1]
     pair = None
+    if act not in EXPERT_ACTIVATIONS:
+        raise KernelError(f"experts_product: activation {act!r} (one of {sorted(filter(None, EXPERT_ACTIVATIONS))})")
     if gated is not None:
-        if gelu or J % 2:
+        if act or J % 2:
             raise KernelError(f"experts_product: a gated activation over {J} rows in pairs, and no other activation")
         pair = _activation_args(gated)
     _need(out, "experts_product.out", (x.dtype, _F32), (None, J // 2 if pair else J))
@@ -1483,7 +1607,7 @@ def experts_product(x, w, out, seg, a_rows, o_rows, row_weight=None, gelu=False,
     if row_weight is not None:
         _need(row_weight, "experts_product.row_weight", _F32, (P,))
     _grouped("experts_product", x, K, 0, w, J * K, K, out, J // 2 if pair else J, 0, P, J, K, E, seg=seg, a_rows=a_rows,
-             o_rows=o_rows, row_weight=row_weight, act=1 if gelu else 0, rows_bound=P, force_simt=force_simt,
+             o_rows=o_rows, row_weight=row_weight, act=EXPERT_ACTIVATIONS[act], rows_bound=P, force_simt=force_simt,
              w_packed=packed, pair=pair)
 
 

@@ -19,7 +19,7 @@ import torch
 
 from ..kernels import ops
 from ..parts.base import Part
-from ..parts.linear import Matrix, linear, as_delta, as_rows
+from ..parts.linear import Matrix, linear, as_delta, as_rows, InjectedDelta
 from ..weights.source import TensorSpec
 
 
@@ -27,37 +27,70 @@ from ..weights.source import TensorSpec
 class LayerRun:
     block: int     # index into DecoderModel.blocks
     cache: int     # index of the cache layer it uses
+    opens: int | None = None     # the pass of the looped layers (LoopInputs) that this run opens
 
 
 class TokenEmbedding(Part):
-    """x[n, :] = scale * E[id[n], :] (crates/synaptix-ops/src/embed/token_embed.rs:4-15; the reference has no scale)."""
+    """x[n, :] = scale * E[id[n], :] (crates/synaptix-ops/src/embed/token_embed.rs:4-15; the reference has no scale).
+    sinusoid_base: a sinusoidal vector of the token's position p is added, with f_i = base^(-2 i / hidden) sin(p f_i) at
+    column 2 i and cos(p f_i) at column 2 i + 1 (None: none)."""
     capturable = True
 
-    def __init__(self, name: str, vocab: int, hidden: int, scale: float = 1.0):
+    def __init__(self, name: str, vocab: int, hidden: int, scale: float = 1.0, sinusoid_base: float | None = None):
         self.name, self.vocab, self.hidden, self.scale = name, vocab, hidden, float(scale)
-        self.table = None
+        self.sinusoid_base = sinusoid_base
+        self.table = self.rates = None
 
     def tensor_specs(self):
         return {self.name: TensorSpec((self.vocab, self.hidden), "table")}
 
     def load(self, get):
         self.table = Matrix(get(self.name))       # (a tied output head multiplies with the same matrix)
+        if self.sinusoid_base is not None:
+            i = torch.arange((self.hidden + 1) // 2, dtype=torch.float64)
+            self.rates = (float(self.sinusoid_base) ** (-2.0 * i / self.hidden)).to(self.table.device)
 
-    def forward(self, ids):
+    def forward(self, ids, positions=None, keep=None):
+        """positions [N] int32: of the rows' tokens (read with sinusoid_base); keep [N, hidden] float: gets the rows too."""
         resid = torch.empty((ids.shape[0], self.hidden), dtype=torch.float32, device=ids.device)
-        if self.scale == 1.0:
+        if self.rates is not None or keep is not None:
+            ops.embed(self.table.data, ids, resid, self.scale,
+                      sinusoid=None if self.rates is None else (self.rates, positions), keep=keep)
+        elif self.scale == 1.0:
             ops.embed(self.table.data, ids, resid)
         else:
             ops.embed(self.table.data, ids, resid, self.scale)
         return resid
 
 
-class OutputHead(Part):
-    """logits = h . W^T in float; tied: W is the embedding table
-    (crates/synaptix-models/llm/common/src/model.rs:757-764)."""
+class LoopInputs(Part):
+    """What layers that run several times in a row get before each pass t = 0, 1, ...: the vector `name`[t] ([times, hidden]),
+    and before every pass but the first the embedding's output once more.  A run of the schedule that opens a pass says so
+    (LayerRun.opens); its first norm adds both (parts.linear.InjectedDelta)."""
     capturable = True
 
-    def __init__(self, name: str, vocab: int, hidden: int, tied_to: TokenEmbedding | None = None):
+    def __init__(self, name: str, times: int, hidden: int):
+        self.name, self.times, self.hidden = name, int(times), hidden
+        self.steps = None
+
+    def tensor_specs(self):
+        return {self.name: TensorSpec((self.times, self.hidden), "bias")}
+
+    def load(self, get):
+        self.steps = get(self.name).float().contiguous()
+
+    def add_to(self, pending, t, resid, embedded):
+        return InjectedDelta(pending, embedded if t > 0 else None, self.steps[t], resid.shape)
+
+
+class OutputHead(Part):
+    """logits = h . W^T in float; tied: W is the embedding table
+    (crates/synaptix-models/llm/common/src/model.rs:757-764).  softcap: logits <- cap tanh(logits / cap)."""
+    capturable = True
+
+    def __init__(self, name: str, vocab: int, hidden: int, tied_to: TokenEmbedding | None = None,
+                 softcap: float | None = None):
+        self.point = ("softcap", float(softcap)) if softcap else None
         self.name, self.vocab, self.hidden, self.tied_to = name, vocab, hidden, tied_to
         self.weight = None
 
@@ -72,17 +105,17 @@ class OutputHead(Part):
         self.weight = self.tied_to.table if self.tied_to is not None else Matrix(get(self.name))
 
     def forward(self, h):
-        return linear(h, self.weight, torch.float32)
+        return linear(h, self.weight, torch.float32, point=self.point)
 
 
 class DecoderModel:
     def __init__(self, config, embedding: TokenEmbedding, blocks: list, schedule: list, final_norm, head: OutputHead,
-                 streams: int | None = None):
-        """streams: the residual runs in this many copies [N, streams, hidden] that all start as the embedding
+                 streams: int | None = None, loop: LoopInputs | None = None):
+        """loop: what the runs that open a pass of looped layers add to the residual.  streams: the residual runs in this many copies [N, streams, hidden] that all start as the embedding
         (blocks that read and write them: parts.HyperConnectionBlock; the final norm gets their sum); None: one
         plain residual [N, hidden]."""
         self.config = config
-        self.streams = streams
+        self.streams, self.loop = streams, loop
         self.embedding, self.blocks, self.schedule = embedding, list(blocks), list(schedule)
         self.final_norm, self.head = final_norm, head
         self.vocab, self.hidden = embedding.vocab, embedding.hidden
@@ -91,6 +124,8 @@ class DecoderModel:
         for run in self.schedule:
             if not (0 <= run.block < len(self.blocks)):
                 raise ValueError(f"schedule names block {run.block}; there are {len(self.blocks)}")
+            if run.opens is not None and (loop is None or streams is not None or not 0 <= run.opens < loop.times):
+                raise ValueError(f"a run that opens pass {run.opens} of looped layers without inputs for it")
         # the first run that names a cache owns (writes) it
         seen, self._owner = set(), []
         for run in self.schedule:
@@ -102,7 +137,7 @@ class DecoderModel:
 
     # ------------------------------------------------------------------ weights
     def _parts(self):
-        return [self.embedding] + self.blocks + [self.final_norm, self.head]
+        return [self.embedding] + self.blocks + [self.final_norm, self.head] + ([] if self.loop is None else [self.loop])
 
     def tensor_specs(self) -> dict:
         specs = {}
@@ -147,7 +182,13 @@ class DecoderModel:
     def forward(self, ctx, tokens, want_rows, cache) -> torch.Tensor:
         """tokens [N] int32 and want_rows [n] int32 (or None) on the device; returns logits [n, vocab] float."""
         with ops.stream_scope():     # one stream for the whole pass, asked for once
-            resid = self.embedding.forward(tokens)
+            embedded = None
+            if any(run.opens for run in self.schedule):       # (a pass behind the first: the embedding's output once more)
+                embedded = torch.empty((tokens.shape[0], self.hidden), dtype=torch.float32, device=tokens.device)
+            if embedded is None and getattr(self.embedding, "rates", None) is None:
+                resid = self.embedding.forward(tokens)
+            else:
+                resid = self.embedding.forward(tokens, ctx.tok_pos, embedded)
             if self.streams is not None:
                 x0, resid = resid, torch.empty((tokens.shape[0], self.streams, self.hidden), dtype=torch.float32,
                                                device=tokens.device)
@@ -155,6 +196,8 @@ class DecoderModel:
             pending = None
             for run, owner in zip(self.schedule, self._owner):
                 block = self.blocks[run.block]
+                if run.opens is not None:
+                    pending = self.loop.add_to(pending, run.opens, resid, embedded)
                 if not block.takes_deferred_product:
                     pending = as_delta(pending)      # a product that the last block left for a norm to take in
                 pending = block.forward(resid, pending, ctx, cache.layer_view(run.cache), owner)

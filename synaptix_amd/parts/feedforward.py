@@ -108,11 +108,13 @@ class RoutedExperts(FeedForward):
 
     The router (32-bit sums of the framework's own product z = W_router h), one of
         "top_logits"  the `top` largest z + bias; weights: softmax over the chosen logits only
-        "scores"      s = softmax(z) over all router outputs; the choice is made on s + correction among the members of
-                      the `keep_groups` best of `n_groups` equal groups of neighbours (a group's score: its largest choice
-                      score); weights: the chosen s themselves (`renorm`: divided by their sum) times `route_scale`
+        "scores"      s = softmax(z) over all router outputs, or with `score="sigmoid"` the sigmoid of each; the choice is
+                      made on s + correction among the members of the `keep_groups` best of `n_groups` equal groups of
+                      neighbours (a group's score: its largest choice score, or with `group_score="two"` the sum of its two
+                      largest); weights: the chosen s themselves (`renorm`: divided by their sum + `renorm_eps`) times
+                      `route_scale`
     The experts, one of
-        ungated       W_down act(W_up h), act the exact GELU
+        ungated       W_down act(W_up h), act the exact GELU or max(z, 0)^2 ("relu_squared")
         gated         W_down act2(W_gate h, W_up h) with an activation of the gated products (ops.ACTIVATIONS; one with a
                       bound as the pair (name, bound))
     `identity`: the router's last `identity` outputs stand for experts without tensors whose result is h itself.
@@ -129,13 +131,14 @@ class RoutedExperts(FeedForward):
     takes_scaled_rows = False
     capturable = True
 
-    ACTIVATIONS = ("gelu",)       # of ungated experts: the exact (erf) form, the products' epilogue
+    ACTIVATIONS = ("gelu", "relu_squared")       # of ungated experts, the products' epilogue (GELU: the exact, erf form)
     ROUTERS = ("top_logits", "scores")
 
     def __init__(self, prefix: str, hidden: int, ff: int, n_experts: int, top: int, activation="gelu",
                  router_bias: bool = True, names=None, *, gated: bool = False, router: str = "top_logits",
                  n_groups: int = 1, keep_groups: int = 1, renorm: bool = False, identity: int = 0, shared=None,
-                 route_scale: float = 1.0, shared_gate: str | None = None):
+                 route_scale: float = 1.0, shared_gate: str | None = None, score: str = "softmax",
+                 group_score: str = "largest", renorm_eps: float = 0.0):
         if router not in self.ROUTERS:
             raise ValueError(f"{prefix}: router {router!r} (one of {self.ROUTERS})")
         if gated:
@@ -157,6 +160,11 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"{prefix}: a factor on the weights comes with the router that scores all outputs")
         if shared_gate is not None and shared is None:
             raise ValueError(f"{prefix}: a gate for a shared expert that is not there")
+        if score not in ("softmax", "sigmoid") or group_score not in ("largest", "two"):
+            raise ValueError(f"{prefix}: scores {score!r} (softmax or sigmoid), groups by {group_score!r} (largest or two)")
+        if router != "scores" and (score, group_score) != ("softmax", "largest"):
+            raise ValueError(f"{prefix}: the kind of scores belongs to the router that scores all outputs")
+        self.score, self.group_score, self.renorm_eps = score, group_score, float(renorm_eps)
         self.route_scale, self.shared_gate = float(route_scale), shared_gate
         self.prefix, self.hidden, self.ff, self.n_experts, self.top = prefix, hidden, ff, n_experts, top
         self.activation, self.gated, self.router = activation, bool(gated), router
@@ -232,7 +240,8 @@ class RoutedExperts(FeedForward):
             logits, shared_gate = logits[:, :self.total], logits[:, self.total:self.total + 1]
         if self.router == "scores":
             ops.route_scores(logits, self.b_router, ids, weights, self.n_groups, self.keep_groups, self.renorm,
-                             self.route_scale)
+                             self.route_scale, sigmoid=self.score == "sigmoid", group_two=self.group_score == "two",
+                             renorm_eps=self.renorm_eps)
         else:
             ops.route_topk(logits.contiguous(), self.b_router, ids, weights)
         seg, tok_of, pair_of, part_of, weight_of = ops.route_sort(ids, weights, self.total)
@@ -243,7 +252,7 @@ class RoutedExperts(FeedForward):
             if self.gated:
                 ops.experts_product(h, self.w_up, mid, real, tok_of, pair_of, gated=self.activation)
             else:
-                ops.experts_product(h, self.w_up, mid, real, tok_of, pair_of, gelu=True)
+                ops.experts_product(h, self.w_up, mid, real, tok_of, pair_of, act=self.activation)
             ops.experts_product(mid, self.w_down, y.view(self.top * N, self.hidden), real, pair_of, part_of,
                                 row_weight=weight_of)
         if self.identity:

@@ -165,9 +165,34 @@ class SummedDeltas:
         return self.scaled().run()
 
 
+class InjectedDelta:
+    """What the residual gets between two layers beside the last sublayer's result `inner` (in any of the forms above, or
+    None): rows [N, hidden] float (or None) and one vector [hidden] float for every row.  A norm that takes it
+    (RmsNorm) adds everything in the pass that norms the rows; everything else asks for `run()`, the sum as one tensor."""
+
+    def __init__(self, inner, rows, vec, shape):
+        """shape: [N, hidden] of the residual."""
+        self.inner, self.rows, self.vec, self.shape = inner, rows, vec, tuple(shape)
+
+    def terms(self):
+        """`inner` as up to two terms of ops.add_scaled_rmsnorm."""
+        d = self.inner
+        if isinstance(d, SummedDeltas) and len(d.terms) <= 2:
+            d = d.scaled()
+        if isinstance(d, ChannelScaledDeltas) and len(d.terms) <= 2:
+            return d.terms
+        d = as_delta(d)
+        return [] if d is None else [(d, None)]
+
+    def run(self):
+        total = torch.zeros(self.shape, dtype=torch.float32, device=self.vec.device)
+        ops.add_scaled_rmsnorm(total, self.terms(), None, 0.0, None, add_rows=self.rows, add_vec=self.vec)
+        return total
+
+
 def as_delta(d):
     """The delta of the residual rows as a tensor (or None), whatever form it arrives in."""
-    if isinstance(d, (DeferredProduct, WeightedDeltas, StreamsWrite, ChannelScaledDeltas, SummedDeltas)):
+    if isinstance(d, (InjectedDelta, DeferredProduct, WeightedDeltas, StreamsWrite, ChannelScaledDeltas, SummedDeltas)):
         return d.run()
     return d
 
@@ -184,8 +209,15 @@ def deferred_product(x, w):
 
 def linear(x, w, out_dtype, point=None):
     """x [M, K] in the activation type, w a Matrix [N, K]; a weight kept in 32-bit takes the 32-bit product.
-    point: an activation that the product applies to its sums before it stores them (ops.POINT_ACTIVATIONS)."""
+    point: an activation that the product applies to its sums before it stores them (ops.POINT_ACTIVATIONS), or
+    ("softcap", cap) with a float result (a pass of its own behind the products that have no such epilogue)."""
     w = _matrix(w)
+    if ops.point_code(point) == ops.POINT_SOFTCAP and not (_use_packed(x, w) and out_dtype == torch.float32):
+        if out_dtype != torch.float32:
+            raise TypeError("linear: a soft cap comes with a float result")
+        out = linear(x, w, out_dtype)
+        ops.soft_cap(out, float(point[1]))
+        return out
     if _use_packed(x, w) and out_dtype in (torch.bfloat16, torch.float32):
         out = torch.empty((x.shape[0], w.shape[0]), dtype=out_dtype, device=x.device)
         if isinstance(x, ScaledRows):

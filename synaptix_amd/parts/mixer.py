@@ -30,6 +30,13 @@ class Mixer(Part):
     or as partial sums [S, N, hidden] that the following norm adds up.
     """
 
+    # True: the mixer is a fused projection of h, something in between, and one output product without a bias, and can share
+    # both products with a mixer beside it (ParallelMixers): it then has
+    #   input_rows(get) -> the projection's matrix;  load_inner(get, scale) -> everything but the two products, with a factor
+    #   on its result;  output_matrix(get);  inner_width, the values it hands the output product;  and
+    #   inner(proj, o, ctx, cache, owner): from its columns of the projection's float rows to its columns of o [N, inner_width]
+    joins = False
+
     # True: `h` may arrive as parts.linear.ScaledRows (rows whose norm a product over packed weights finishes)
     # and the returned delta may be a parts.linear.DeferredProduct; False (the default): plain tensors both ways
     takes_scaled_rows = False
@@ -272,6 +279,7 @@ class GatedWindowAttention(Mixer):
         self.score_softcap = float(score_softcap) if score_softcap else 0.0
         self.names = dict(self.NAMES, **(names or {}))
         self.w_in = self.w_o = self.b_in = self.b_o = self.q_gain = self.k_gain = self.sinks = None
+        self.inner_width, self.result_scale = self.nh * self.vdim, 1.0
         self._terms = None
 
     def _n(self, key, bias=False):
@@ -305,10 +313,24 @@ class GatedWindowAttention(Mixer):
         specs.update(self.position.tensor_specs())
         return specs
 
+    @property
+    def joins(self):
+        return not self.out_bias
+
+    def input_rows(self, get):
+        """One product for q, k, v and the gate: rows of the matrices one after another."""
+        return torch.cat([get(self._n(k)) for k, _ in self._widths()], 0)
+
+    def output_matrix(self, get):
+        return get(self._n("o"))
+
     def load(self, get):
-        # one product for q, k, v and the gate: rows of the matrices one after another
-        self.w_in = _projection(_whole_fragments(torch.cat([get(self._n(k)) for k, _ in self._widths()], 0)))
-        self.w_o = _projection(get(self._n("o")))
+        self.w_in = _projection(_whole_fragments(self.input_rows(get)))
+        self.w_o = _projection(self.output_matrix(get))
+        self.load_inner(get)
+
+    def load_inner(self, get, scale: float = 1.0):
+        self.result_scale = float(scale)
         if self.bias:
             self.b_in = torch.cat([get(self._n(k, True)).float() for k, _ in self._biased()]).contiguous()
         if self.out_bias:
@@ -340,27 +362,34 @@ class GatedWindowAttention(Mixer):
         return self._terms
 
     def forward(self, h, ctx, cache, owner=True):
-        N, act = h.shape[0], h.dtype
+        proj = linear(h, self.w_in, torch.float32)          # [N, q | k | v | gate] float (q | gate with shared_kv)
+        o = torch.empty((h.shape[0], self.inner_width), dtype=h.dtype, device=h.device)
+        self.inner(proj, o, ctx, cache, owner)
+        if self.b_o is None:
+            return deferred_product(o, self.w_o)
+        return WeightedDeltas([(linear_for_sum(o, self.w_o), 1.0, self.b_o)])
+
+    def inner(self, proj, o, ctx, cache, owner=True):
+        N, act = o.shape[0], o.dtype
         if owner == self.shared_kv:
             raise ValueError(f"{self.prefix}: a layer {'without' if owner else 'with'} keys and values of its own was "
                              f"scheduled as the cache's {'owner' if owner else 'reader'}")
         cap = self.position.capacity
         if cap is not None and ctx.max_position >= cap:
             raise ValueError(f"position {ctx.max_position} is beyond the position encoding's capacity {cap}")
-        proj = linear(h, self.w_in, torch.float32)          # [N, q | k | v | gate] float (q | gate with shared_kv)
-        q = torch.empty((N, self.nh * self.dim), dtype=act, device=h.device)
+        q = torch.empty((N, self.nh * self.dim), dtype=act, device=o.device)
         table = ctx.page_table(cache.group)
         ops.window_intake(proj, self.b_in, q, cache.k_pages, cache.v_pages, table, ctx.tok_seq, ctx.tok_pos,
                           self.q_gain, self.k_gain, self.qk_norm_eps or 0.0, self.nh, self.nkv, self.dim, self.vdim,
-                          write_kv=owner, rotation=self.position.tables(h.device), pairs=self.position.pairing == "pairs",
+                          write_kv=owner, rotation=self.position.tables(o.device), pairs=self.position.pairing == "pairs",
                           norm_whole=self.qk_norm_whole, values_are_keys=self.values_are_keys, q_temp=self.q_temp)
-        o = torch.empty((N, self.nh * self.vdim), dtype=act, device=h.device)
         at = sum(n for _, n in self._biased())
         gate = proj[:, at:at + self._widths()[-1][1]] if self.gate else None
         how = dict(window=self.window or 0, keep_first=self.keep_first, sink_one=self.sink_one, gate=gate,
-                   gate_per_head=self.gate == "head", sinks=self.sinks, chunk=self.chunk or 0,
-                   **self._score_terms(h.device))
-        if act == torch.bfloat16 and not ctx.one_token_each and ops.window_prefill_takes(self.dim, self.vdim):
+                   gate_per_head=self.gate == "head", sinks=self.sinks, chunk=self.chunk or 0, out_scale=self.result_scale,
+                   **self._score_terms(o.device))
+        if (act == torch.bfloat16 and not ctx.one_token_each and ops.window_prefill_takes(self.dim, self.vdim)
+                and o.stride(0) % 4 == 0):
             # prompts in bf16: tiles of queries on the matrix cores
             ops.window_attention_prefill_bf16(q, cache.k_pages, cache.v_pages, table, ctx.seq_start, ctx.seq_past, o,
                                               self.scale, self.nh, self.nkv, self.dim, self.vdim, **how)
@@ -368,9 +397,6 @@ class GatedWindowAttention(Mixer):
             # 32-bit, single tokens, and head sizes that the tiles do not take: a wave (or eight) for each (token, head)
             ops.window_attention(q, cache.k_pages, cache.v_pages, table, ctx.tok_seq, ctx.tok_pos, o, self.scale, self.nh,
                                  self.nkv, self.dim, self.vdim, **how)
-        if self.b_o is None:
-            return deferred_product(o, self.w_o)
-        return WeightedDeltas([(linear_for_sum(o, self.w_o), 1.0, self.b_o)])
 
 
 class DifferentialAttention(Mixer):
@@ -485,13 +511,22 @@ class DifferentialAttention(Mixer):
 
 class ParallelMixers(Mixer):
     """Several mixers side by side that read the same input; the result is sum_i scale_i * mixer_i(h).  Each keeps
-    what it needs for a sequence: the cache need is the tuple of theirs, and so is the cache view."""
-    takes_scaled_rows = False
+    what it needs for a sequence: the cache need is the tuple of theirs, and so is the cache view.
+
+    Where all of them say that they join (Mixer.joins), they share one input projection and one output product:
+    sum_i scale_i W_i o_i = [W_1 | W_2 | ...] [scale_1 o_1 ; scale_2 o_2 ; ...], with the factors applied in 32-bit where each
+    writes its columns of the row.  The row is padded with zeros to a multiple of 32, which the output matrix then has too."""
 
     def __init__(self, mixers: list, scales: list):
         if len(mixers) != len(scales) or not mixers:
             raise ValueError("one scale for each of the mixers")
         self.mixers, self.scales = list(mixers), [float(s) for s in scales]
+        self.joined = all(getattr(m, "joins", False) for m in self.mixers)
+        self.w_in = self.w_o = None
+
+    @property
+    def takes_scaled_rows(self):
+        return self.joined
 
     @property
     def capturable(self):
@@ -504,8 +539,23 @@ class ParallelMixers(Mixer):
         return specs
 
     def load(self, get):
-        for m in self.mixers:
-            m.load(get)
+        if not self.joined:
+            for m in self.mixers:
+                m.load(get)
+            return
+        rows = [m.input_rows(get) for m in self.mixers]
+        self.columns = []             # of the projection's rows: each mixer's first, and how many
+        for r in rows:
+            self.columns.append((sum(n for _, n in self.columns), r.shape[0]))
+        self.w_in = _projection(_whole_fragments(torch.cat(rows, 0)))
+        outs = [m.output_matrix(get) for m in self.mixers]
+        spare = -sum(o.shape[1] for o in outs) % 32
+        if spare:
+            outs.append(torch.zeros((outs[0].shape[0], spare), dtype=outs[0].dtype, device=outs[0].device))
+        self.spare = spare
+        self.w_o = _projection(torch.cat(outs, 1).contiguous())
+        for m, s in zip(self.mixers, self.scales):
+            m.load_inner(get, s)
 
     def check(self, dtype):
         for m in self.mixers:
@@ -515,6 +565,15 @@ class ParallelMixers(Mixer):
         return tuple(m.cache_need() for m in self.mixers)
 
     def forward(self, h, ctx, cache, owner=True):
+        if self.joined:
+            proj = linear(h, self.w_in, torch.float32)
+            new = torch.zeros if self.spare else torch.empty
+            o = new((h.shape[0], self.w_o.shape[1]), dtype=h.dtype, device=h.device)
+            at = 0
+            for m, c, (first, n) in zip(self.mixers, cache, self.columns):
+                m.inner(proj[:, first:first + n], o[:, at:at + m.inner_width], ctx, c, owner)
+                at += m.inner_width
+            return deferred_product(o, self.w_o)
         terms = []
         for m, s, c in zip(self.mixers, self.scales, cache):
             y = m.forward(h, ctx, c, owner)

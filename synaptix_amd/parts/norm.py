@@ -13,7 +13,7 @@ import torch
 from ..kernels import ops
 from ..weights.source import TensorSpec
 from .base import Part
-from .linear import DeferredProduct, ScaledRows, ChannelScaledDeltas, SummedDeltas
+from .linear import DeferredProduct, ScaledRows, ChannelScaledDeltas, SummedDeltas, InjectedDelta
 
 
 class RmsNorm(Part):
@@ -35,9 +35,26 @@ class RmsNorm(Part):
     def load(self, get):
         self.gain = get(self.name)
 
+    def _runs_product(self, resid, delta, out_dtype, rows):
+        """Whether this norm takes `delta`, a product that has not been run, in as its epilogue's residual sum."""
+        return (isinstance(delta, DeferredProduct) and rows is None and out_dtype == torch.bfloat16
+                and delta.shape == tuple(resid.shape) and self.dim % 16 == 0)
+
     def add_apply(self, resid, delta, out_dtype, rows=None):
         """resid [N, dim] float: with rows None, resid += delta (if any) in place and every row is
         normed; with rows [n] int32 only those rows of resid + delta are normed and resid is kept."""
+        more = (None, None)
+        if isinstance(delta, InjectedDelta):
+            # the residual gets rows or a vector beside the last sublayer's result: added in the pass that norms it
+            if self.gain_offset == 0.0 and not self._runs_product(resid, delta.inner, out_dtype, rows):
+                n = resid.shape[0] if rows is None else rows.shape[0]
+                out = torch.empty((n, self.dim), dtype=out_dtype, device=resid.device)
+                ops.add_scaled_rmsnorm(resid, delta.terms(), self.gain, self.eps, out, rows, delta.rows, delta.vec)
+                return out
+            if self._runs_product(resid, delta.inner, out_dtype, rows):
+                delta, more = delta.inner, (delta.rows, delta.vec)
+            else:
+                delta = delta.run()
         if isinstance(delta, SummedDeltas):
             # a sublayer's result in several terms (routed experts' partial sums, a gated shared expert)
             delta = delta.scaled() if len(delta.terms) <= 2 else delta.run()
@@ -52,11 +69,10 @@ class RmsNorm(Part):
         if isinstance(delta, DeferredProduct):
             # a product over packed weights for few rows: it adds its sums into resid itself and leaves the rows with
             # the gain and the row statistic in groups; the product that follows applies the row's factor
-            if (rows is None and out_dtype == torch.bfloat16 and delta.shape == tuple(resid.shape)
-                    and self.dim % 16 == 0):
+            if self._runs_product(resid, delta, out_dtype, rows):
                 xs = torch.empty(resid.shape, dtype=torch.bfloat16, device=resid.device)
                 ss = torch.empty((resid.shape[0], self.dim // 16), dtype=torch.float32, device=resid.device)
-                ops.gemm_packed(delta.x, delta.packed, None, resid_norm=(resid, self.gain, self.gain_offset, xs, ss))
+                ops.gemm_packed(delta.x, delta.packed, None, resid_norm=(resid, self.gain, self.gain_offset, xs, ss, *more))
                 return ScaledRows(xs, ss, self.eps, resid, self)
             delta = delta.run()
         n = resid.shape[0] if rows is None else rows.shape[0]

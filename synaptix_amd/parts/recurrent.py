@@ -14,6 +14,10 @@ HeadDeltaMixer: the delta rule with one decay a head, exp(-exp(A) softplus(W_a h
 by its root mean square, times a gain, times silu(W_g h); everything in front of the cell is one fused projection
 [q | k | v | gate | step | decay].
 
+GatedLinearAttention: no convolution and no correction, S <- diag(g) S + k v^T, with a decay for every (head, key channel)
+g = sigmoid(W_a2 W_a1 h + bias)^(1 / tau); each head's read-out is divided by its root mean square, times a gain, times
+silu(W_g h); the fused projection is [q | k | v | gate | the narrow middle W_a1 h].
+
 Step sizes, decays, gates, unit norms, states and everything between the projections and the output product are 32-bit
 in both engine types.  A sequence's state (the matrix, and the convolution's last inputs) starts at zero when its slot
 is taken and is carried from step to step.
@@ -263,3 +267,95 @@ class HeadDeltaMixer(Mixer):
         o = torch.empty((N, E), dtype=h.dtype, device=proj.device)
         ops.head_norm_gate(raw, self.gain, self.norm_eps, proj[:, C:], o, H, self.vdim, silu=True)
         return deferred_product(o, self.w_o)
+
+
+class GatedLinearAttention(Mixer):
+    """Gated linear attention (csrc/recurrent.hip).  Tensors: prefix + "q", "k" [heads x dim, hidden], "v", "g"
+    [heads x vdim, hidden], "a1" [rank, hidden], "a2" [heads x dim, rank], "a2.b" [heads x dim], "norm" [vdim], "o"; the
+    size of the narrow middle is what the stored tensors say (set_rank names it for random weights)."""
+    takes_scaled_rows = True      # (the products at both ends take a norm's halves: parts.linear)
+    capturable = True
+    joins = True
+
+    NAMES = {"q": "q", "k": "k", "v": "v", "g": "g", "a1": "a1", "a2": "a2", "a_bias": "a2.b", "norm": "norm", "o": "o"}
+
+    def __init__(self, prefix: str, hidden: int, n_heads: int, dim: int, vdim: int, tau: float, *, norm_eps: float,
+                 q_scale: float | None = None, names: dict | None = None):
+        if not tau > 0.0:
+            raise ValueError(f"{prefix}: tau {tau} must be positive")
+        self.prefix, self.hidden = prefix, hidden
+        self.nh, self.dim, self.vdim, self.tau, self.norm_eps = n_heads, dim, vdim, float(tau), float(norm_eps)
+        self.q_scale = float(q_scale) if q_scale is not None else dim ** -0.5
+        self.names = dict(self.NAMES, **(names or {}))
+        self.rank = None
+        self.inner_width = n_heads * vdim
+        self.w_in = self.w_o = self.a2 = self.a_bias = self.gain = None
+
+    def _n(self, key):
+        return self.prefix + self.names[key]
+
+    def _rows(self):
+        """The fused projection's pieces, in their order."""
+        return [("q", self.nh * self.dim), ("k", self.nh * self.dim), ("v", self.nh * self.vdim), ("g", self.nh * self.vdim),
+                ("a1", self.rank)]
+
+    def set_rank(self, rank: int):
+        self.rank = int(rank)
+
+    def tensor_specs(self):
+        specs = {self._n(k): TensorSpec((n, self.hidden)) for k, n in self._rows()}
+        specs.update({self._n("a2"): TensorSpec((self.nh * self.dim, self.rank)),
+                      self._n("a_bias"): TensorSpec((self.nh * self.dim,), "bias"),
+                      self._n("norm"): TensorSpec((self.vdim,), "gain"),
+                      self._n("o"): TensorSpec((self.hidden, self.nh * self.vdim))})
+        return specs
+
+    def input_rows(self, get):
+        return torch.cat([get(self._n(k)) for k, _ in self._rows()], 0)
+
+    def output_matrix(self, get):
+        return get(self._n("o"))
+
+    def load(self, get):
+        self.w_in = _projection(_whole_fragments(self.input_rows(get)))
+        self.w_o = _projection(self.output_matrix(get))
+        self.load_inner(get)
+
+    def load_inner(self, get, scale: float = 1.0):
+        a1, a2 = get(self._n("a1")), get(self._n("a2"))
+        if a2.shape[1] != a1.shape[0]:
+            raise ValueError(f"{self.prefix}: a narrow middle of {a1.shape[0]} values meets a matrix for {a2.shape[1]}")
+        self.rank = a1.shape[0]
+        self.a2 = a2.float().T.contiguous()               # [rank, heads x dim]: neighbouring channels side by side
+        self.a_bias = get(self._n("a_bias")).float().contiguous()
+        self.gain = (get(self._n("norm")).float() * scale).repeat(self.nh).contiguous()     # one gain for all heads
+
+    def cache_need(self):
+        return StateNeed((self.nh, self.dim, self.vdim))
+
+    def check(self, dtype):
+        if self.dim > ops.SCAN_MAX_ROWS or self.vdim > ops.GATED_LINEAR_MAX_VDIM:
+            raise ValueError(f"{self.prefix}: keys of {self.dim} values (at most {ops.SCAN_MAX_ROWS}), values of {self.vdim} "
+                             f"(at most {ops.GATED_LINEAR_MAX_VDIM})")
+
+    def forward(self, h, ctx, cache, owner=True):
+        proj = linear(h, self.w_in, torch.float32)          # [N, q | k | v | gate | middle] float
+        o = torch.empty((h.shape[0], self.inner_width), dtype=h.dtype, device=h.device)
+        self.inner(proj, o, ctx, cache, owner)
+        return deferred_product(o, self.w_o)
+
+    def inner(self, proj, o, ctx, cache, owner=True):
+        K, E, at = self.nh * self.dim, self.nh * self.vdim, 0
+        cols = []
+        for n in (K, K, E, E, self.rank):
+            cols.append(proj[:, at:at + n])
+            at += n
+        q, k, v, gate, mid = cols
+        if ctx.one_token_each:
+            ops.gated_linear_step(q, k, v, mid, self.a2, self.a_bias, self.q_scale, self.tau, cache.state, ctx.seq_start,
+                                  ctx.seq_slot, self.gain, self.norm_eps, gate, o, self.nh, self.dim, self.vdim)
+            return
+        raw = torch.empty((o.shape[0], E), dtype=torch.float32, device=o.device)
+        ops.gated_linear_scan(q, k, v, mid, self.a2, self.a_bias, self.q_scale, self.tau, cache.state, ctx.seq_start,
+                              ctx.seq_slot, raw, self.nh, self.dim, self.vdim, scratch=ctx.scratch)
+        ops.head_norm_gate(raw, self.gain, self.norm_eps, gate, o, self.nh, self.vdim, silu=True)

@@ -131,7 +131,7 @@ def test_router_and_experts(N, W, F, E, top, dtype):
     for w_up, w_down in kept:
         for force in (0, 1, 2, 3):      # by size; plain FMA; the matrix cores without LDS, 16 and 64 outputs a wave
             mid = torch.empty((N * top, F), dtype=dtype, device=DEV)
-            ops.experts_product(dev(h, dtype), w_up, mid, seg, tok_of, pair_of, gelu=True, force_simt=force)
+            ops.experts_product(dev(h, dtype), w_up, mid, seg, tok_of, pair_of, act="gelu", force_simt=force)
             y = torch.empty((top, N, W), dtype=torch.float32, device=DEV)
             ops.experts_product(mid, w_down, y.view(top * N, W), seg, pair_of, part_of, row_weight=weight_of,
                                 force_simt=force)
