@@ -210,11 +210,11 @@ def design_configs(design, size, window, context):
     layers have latent attention (a latent of 512, 64 rotated values, unrotated keys and values of the head size; every
     second layer with the window) and a mixture of experts whose active width equals the dense feed-forward's."""
     from synaptix_amd import Qwen3Config
-    from synaptix_amd.config import BizipelConfig, KamivikConfig, RepolixConfig, NilepelConfig, PizunexConfig
+    from synaptix_amd.config import BizipelConfig, KamivikConfig, RepolixConfig, NilepelConfig, PizunexConfig, SunosunConfig
     L, W, nh, nkv, hd, ff, V = SIDE_BY_SIDE_SIZES[size]
     qwen = Qwen3Config.from_dict(dict(_COMMON, num_hidden_layers=L, hidden_size=W, num_attention_heads=nh,
                                       num_key_value_heads=nkv, head_dim=hd, intermediate_size=ff, vocab_size=V,
-                                      tie_word_embeddings=design == "bizipel", max_position_embeddings=context))
+                                      tie_word_embeddings=design in ("bizipel", "sunosun"), max_position_embeddings=context))
     if design == "repolix":
         E, I, top, eff = repolix_experts(size)
         mlp = {"kind": "moe", "expert": {"ff": eff, "limit": 7.0}, "shared": {"ff": eff, "limit": 7.0},
@@ -248,6 +248,21 @@ def design_configs(design, size, window, context):
         nil = NilepelConfig.from_dict({"architecture": "Nilepel", "vocab": V, "width": W, "norm": {"eps": 1e-6},
                                        "embedding": {"scale": float(W) ** 0.5}, "layers": layers})
         return qwen, nil
+    if design == "sunosun":
+        E, _, top, eff = repolix_experts(size)
+        moe = {"kind": "moe", "expert": {"ff": eff}, "shared": {"ff": eff},
+               "router": {"experts": E, "top": top, "scale": 2.0, "groups": {"count": 2, "keep": 1}}}
+        dense = {"kind": "dense", "ff": ff}
+        linear = {"heads": nh, "dim": hd, "vdim": hd, "tau": 16.0}
+        both = {"left": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5},
+                "right": dict(linear, heads=max(1, nh // 2)), "left_scale": 0.5, "right_scale": 0.75}
+        sun = SunosunConfig.from_dict({"architecture": "Sunosun", "vocab": V, "width": W, "norm": {"eps": 1e-6},
+                                       "embedding": {"scale": 4.0}, "logit_softcap": 30.0, "middle_rank": 16,
+                                       "loop": {"start": 1, "stop": 2, "times": 2},
+                                       "layers": [{"type": "gla", "mixer": linear, "mlp": dense},
+                                                  {"type": "gla", "mixer": linear, "mlp": moe},
+                                                  {"type": "parallel", "mixer": both, "mlp": dense}]})
+        return qwen, sun
     if design == "pizunex":
         mixers = {"delta": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "conv": 4},
                   "attention": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "softcap": 50.0,
@@ -322,6 +337,14 @@ def designs_side_by_side(args) -> int:
                 one = 3 * 2 * eff * cfg.width
                 touched = E * (1.0 - (1.0 - top / E) ** B)
                 weight_bytes -= int(sum(1 for l in cfg.layers if l.mlp.kind == "moe") * (E - touched) * one)
+            if design == "sunosun":
+                # likewise; and the looped layer's tensors are read in each of its passes
+                E, _, top, eff = repolix_experts(size)
+                touched = E * (1.0 - (1.0 - top / E) ** B)
+                block = sum(2 * int(torch.Size(sp.shape).numel()) for n, sp in eng.model.tensor_specs().items()
+                            if n.startswith(f"l{cfg.loop.start}."))
+                block -= int((E - touched) * 2 * 2 * eff * cfg.width)
+                weight_bytes += (cfg.loop.times - 1) * block - int((E - touched) * 2 * 2 * eff * cfg.width)
             g = torch.Generator().manual_seed(0)
             prompt = torch.randint(0, cfg.vocab_size, (P,), generator=g).tolist()
             times = []
@@ -392,7 +415,7 @@ def main() -> int:
                     help="the longest sequence (positions and cache a sequence; the contract's run has 8,192)")
     ap.add_argument("--no-points", action="store_true", help="skip decode at batch 1 and 64")
     ap.add_argument("--no-graph", action="store_true", help="launch every kernel of a decode step from the host")
-    ap.add_argument("--design", default=None, choices=["bizipel", "kamivik", "repolix", "nilepel", "pizunex"],
+    ap.add_argument("--design", default=None, choices=["bizipel", "kamivik", "repolix", "nilepel", "pizunex", "sunosun"],
                     help="another run than the default one: this design beside the Qwen3 decoder at equal layer sizes")
     ap.add_argument("--sizes", default="small,mid,large", help="with --design: which of small, mid, large")
     ap.add_argument("--window", type=int, default=1024, help="with --design: the keys a query of the new design sees")

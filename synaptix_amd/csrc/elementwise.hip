@@ -14,17 +14,17 @@ SYN_DEFINE_ERROR_CHANNEL
 // ------------------------------------------------------------------ embedding
 // resid[n, :] = scale * table[ids[n], :] widened to float.  Ids are checked on the host.
 // pos.rates != null: a sinusoidal position vector is added, sin(p f_i) at column 2 i and cos(p f_i) at 2 i + 1 for the token
-// at position p; the angle is taken in 64-bit and reduced to one turn there, so that it is as good at any position as near 0.
+// at position p; the angle is taken in 64-bit, in turns, and whole turns are dropped there, so that it is as good at any
+// position as near 0.
 // keep != null: the rows once more (resid is written on by the layers).
 struct EmbedPositions {
-  const double* rates;   // [(H + 1) / 2] f_i, or null
+  const double* rates;   // [(H + 1) / 2] f_i / (2 pi), or null
   const int* pos;        // [tokens]
 };
-__device__ __forceinline__ float embed_position(const EmbedPositions& p, int n, int col) {
-  constexpr double TURN = 6.283185307179586;
-  double a = (double)p.pos[n] * p.rates[col / 2];
-  a -= TURN * rint(a / TURN);
-  return col % 2 ? cosf((float)a) : sinf((float)a);
+__device__ __forceinline__ void embed_position(const EmbedPositions& p, int n, int pair, float& s, float& c) {
+  double turns = (double)p.pos[n] * p.rates[pair];
+  turns -= rint(turns);
+  sincospif((float)(2.0 * turns), &s, &c);
 }
 
 template <typename T>
@@ -35,7 +35,11 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
   float* out = resid + (size_t)n * H;
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
     float v = to_f32<T>(row[i]) * scale;
-    if (p.rates) v += embed_position(p, n, i);
+    if (p.rates) {
+      float s, c;
+      embed_position(p, n, i / 2, s, c);
+      v += i % 2 ? c : s;
+    }
     out[i] = v;
     if (keep) keep[(size_t)n * H + i] = v;
   }
@@ -48,14 +52,18 @@ __global__ void embed_packed_kernel(const bf16* __restrict__ table, const int* _
   const int n = blockIdx.x, id = ids[n];
   const bf16* group = table + (size_t)(id / 16) * H * 16;   // the 16 rows around row id: H / 32 fragments of 512 values
   float* out = resid + (size_t)n * H;
-  for (int c = threadIdx.x; c < H / 8; c += blockDim.x) {   // chunk c: values 8 c .. 8 c + 7 of the row
+  for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < H / 8; c += blockDim.x * gridDim.y) {   // values 8 c .. 8 c + 7 of the row
     const bf16x8 v = *(const bf16x8*)(group + (size_t)(c / 4) * 512 + ((c % 4) * 16 + id % 16) * 8);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      float x = (float)v[e] * scale;
-      if (p.rates) x += embed_position(p, n, c * 8 + e);
-      out[c * 8 + e] = x;
-      if (keep) keep[(size_t)n * H + c * 8 + e] = x;
+    for (int e = 0; e < 8; e += 2) {
+      float x0 = (float)v[e] * scale, x1 = (float)v[e + 1] * scale;
+      if (p.rates) {
+        float s, t;
+        embed_position(p, n, c * 4 + e / 2, s, t);
+        x0 += s, x1 += t;
+      }
+      out[c * 8 + e] = x0, out[c * 8 + e + 1] = x1;
+      if (keep) keep[(size_t)n * H + c * 8 + e] = x0, keep[(size_t)n * H + c * 8 + e + 1] = x1;
     }
   }
 }
@@ -71,7 +79,8 @@ SYN_EXPORT int syn_embed(const void* table, int table_kind, const int* ids, floa
     embed_kernel<float><<<n_tokens, 256, 0, stream>>>((const float*)table, ids, resid, H, scale, p, keep);
   } else if (table_kind == 2) {
     SYN_CHECK(H % 32 == 0, "embed: a table in fragment order has a width that is a multiple of 32, not %d", H);
-    embed_packed_kernel<<<n_tokens, 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale, p, keep);
+    const dim3 grid(n_tokens, rates ? (H / 8 + 63) / 64 : 1);
+    embed_packed_kernel<<<grid, rates ? 64 : 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale, p, keep);
   } else {
     embed_kernel<bf16><<<n_tokens, 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale, p, keep);
   }
@@ -763,6 +772,72 @@ __global__ void add_scaled_rmsnorm_kernel(float* __restrict__ resid, const int* 
   }
 }
 
+// The same with four neighbouring values a lane and a thread's NV groups of them in registers: everything is read once, and a
+// term's partial sums are asked for four at a time.  Widths that are multiples of 4, up to 4096 NV.
+template <typename TOut, int NV>
+__global__ void __launch_bounds__(1024)
+add_scaled_rmsnorm_vec_kernel(float* __restrict__ resid, const int* __restrict__ rows, size_t part_stride,
+                              const float* __restrict__ d1, int parts1, const float* __restrict__ s1,
+                              const float* __restrict__ d2, int parts2, const float* __restrict__ s2,
+                              const float* __restrict__ g1, int g1_stride, const float* __restrict__ g2, int g2_stride,
+                              const float* __restrict__ add_rows, const float* __restrict__ add_vec,
+                              const void* __restrict__ gain, int gain_is_f32, float eps, TOut* __restrict__ out, int H) {
+  __shared__ float red[16];
+  const int r = rows ? rows[blockIdx.x] : blockIdx.x;
+  const float f1 = g1 ? 1.f / (1.f + expf(-g1[(size_t)r * g1_stride])) : 1.f;
+  const float f2 = g2 ? 1.f / (1.f + expf(-g2[(size_t)r * g2_stride])) : 1.f;
+  float* x = resid + (size_t)r * H;
+  const bool write_back = rows == nullptr;
+  f32x4 v[NV];
+  auto add_term = [&](f32x4& to, int i, const float* d, int parts, const float* s, float f) {
+    const float* p = d + (size_t)r * H + i;
+    f32x4 t = {0.f, 0.f, 0.f, 0.f};
+    int k = 0;
+    for (; k + 4 <= parts; k += 4) {
+      f32x4 u[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) u[j] = *(const f32x4*)(p + (k + j) * part_stride);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) t += u[j];
+    }
+    for (; k < parts; ++k) t += *(const f32x4*)(p + k * part_stride);
+    const f32x4 w = s ? *(const f32x4*)(s + i) * f : f32x4{f, f, f, f};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) to[e] = fmaf(w[e], t[e], to[e]);
+  };
+  float ss = 0.f;
+#pragma unroll
+  for (int n = 0; n < NV; ++n) {
+    const int i = (threadIdx.x + n * blockDim.x) * 4;
+    v[n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (i < H) {
+      v[n] = *(const f32x4*)(x + i);
+      if (d1) add_term(v[n], i, d1, parts1, s1, f1);
+      if (d2) add_term(v[n], i, d2, parts2, s2, f2);
+      if (add_rows) v[n] += *(const f32x4*)(add_rows + (size_t)r * H + i);
+      if (add_vec) v[n] += *(const f32x4*)(add_vec + i);
+      if (write_back) *(f32x4*)(x + i) = v[n];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[n][e], v[n][e], ss);
+  }
+  if (out == nullptr) return;         // (uniform)
+  ss = block_sum(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)H + eps);
+  TOut* o = out + (size_t)blockIdx.x * H;
+#pragma unroll
+  for (int n = 0; n < NV; ++n) {
+    const int i = (threadIdx.x + n * blockDim.x) * 4;
+    if (i < H) {
+      typedef TOut out4 __attribute__((ext_vector_type(4)));
+      out4 y;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = from_f32<TOut>(load_gain(gain, gain_is_f32, i + e) * (v[n][e] * inv));
+      *(out4*)(o + i) = y;
+    }
+  }
+}
+
 SYN_EXPORT int syn_add_scaled_rmsnorm(float* resid, int n_rows, const int* rows, int n_out, const float* d1, int parts1,
                                       const float* s1, const float* d2, int parts2, const float* s2, const float* g1,
                                       int g1_stride, const float* g2, int g2_stride, const float* add_rows,
@@ -772,6 +847,24 @@ SYN_EXPORT int syn_add_scaled_rmsnorm(float* resid, int n_rows, const int* rows,
   SYN_CHECK(parts1 >= 1 && parts1 <= 64 && parts2 >= 1 && parts2 <= 64, "add_scaled_rmsnorm: %d and %d partial sums", parts1, parts2);
   SYN_CHECK(out == nullptr || gain != nullptr, "add_scaled_rmsnorm: a norm needs its gain");
   const size_t stride = (size_t)n_rows * H;
+  auto aligned = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  if (H % 4 == 0 && H <= 16384 && aligned(resid) && aligned(d1) && aligned(s1) && aligned(d2) && aligned(s2) &&
+      aligned(add_rows) && aligned(add_vec) && (uintptr_t)out % 16 == 0) {
+    const int nv = H <= 4096 ? 1 : (H <= 8192 ? 2 : 4);
+    const int threads = ((H / 4 + nv - 1) / nv + SYN_WAVE - 1) / SYN_WAVE * SYN_WAVE;
+#define SYN_ASV(T, NV)                                                                                                      \
+  add_scaled_rmsnorm_vec_kernel<T, NV><<<n_out, threads, 0, stream>>>(resid, rows, stride, d1, parts1, s1, d2, parts2, s2, \
+                                                                      g1, g1_stride, g2, g2_stride, add_rows, add_vec,     \
+                                                                      gain, gain_is_f32, eps, (T*)out, H)
+    if (out_is_f32) {
+      if (nv == 1) SYN_ASV(float, 1); else if (nv == 2) SYN_ASV(float, 2); else SYN_ASV(float, 4);
+    } else {
+      if (nv == 1) SYN_ASV(bf16, 1); else if (nv == 2) SYN_ASV(bf16, 2); else SYN_ASV(bf16, 4);
+    }
+#undef SYN_ASV
+    SYN_LAUNCH_CHECK("add_scaled_rmsnorm_vec");
+    return 0;
+  }
   const int block = H >= 4096 ? 1024 : (H >= 1024 ? 512 : 256);
   if (out_is_f32)
     add_scaled_rmsnorm_kernel<float><<<n_out, block, 0, stream>>>(resid, rows, stride, d1, parts1, s1, d2, parts2, s2, g1,

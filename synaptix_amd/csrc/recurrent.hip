@@ -888,6 +888,17 @@ struct GlaArgs {
   int H, D, E;
 };
 
+// log2 of a decay: -softplus(-z) / (tau ln 2), on the hardware's base-2 exponential and logarithm.  With w = 1 + u rounded,
+// log(1 + u) = log w + (u - (w - 1)) / w up to second order in the rounding error, so that decays next to one keep their
+// digits.
+__device__ __forceinline__ float gla_log2_decay(float z, float inv_tau) {
+  constexpr float LOG2E = 1.4426950408889634f;
+  const float y = -z * LOG2E;                                   // softplus(-z) / ln 2 = log2(1 + 2^y)
+  const float u = __builtin_amdgcn_exp2f(y), w = 1.f + u;
+  const float sp = fmaf((u - (w - 1.f)) * LOG2E, __builtin_amdgcn_rcpf(w), __builtin_amdgcn_logf(w));
+  return -(y > 30.f ? y : sp) * inv_tau;
+}
+
 #define GLA_STEP_THREADS 512
 #define GLA_STEP_AHEAD 8     // rows of the state that a thread has under way
 
@@ -905,7 +916,7 @@ gla_step_kernel(GlaArgs a, const float* __restrict__ gain, float eps, const floa
   float* qs = lds;                  // [D]
   float* ks = qs + D;               // [D]
   float* gs = ks + D;               // [D]
-  float* part = gs + D;             // [row groups][E]
+  float* part = gs + D;             // [row groups][E]; before that [rank shares][D]
   const int CL = E / VEC, RG = GLA_STEP_THREADS / CL;      // (the host: E a multiple of VEC, CL at most the threads)
   const int cl = tid % CL, rg = tid / CL;
   const bool on = rg < RG;
@@ -927,13 +938,33 @@ gla_step_kernel(GlaArgs a, const float* __restrict__ gain, float eps, const floa
   else
 #pragma unroll
     for (int e = 0; e < VEC; ++e) v[e] = on ? a.v[tok * a.ld + head * E + cl * VEC + e] : 0.f;
-  for (int d = tid; d < D; d += GLA_STEP_THREADS) {
-    const int hd = head * D + d;
+  // the decays: the middle's values are shared out over as many threads a channel as there are
+  const int shares = GLA_STEP_THREADS / D, share = tid / D, d = tid % D, hd = head * D + d;      // (the host: D at most 256)
+  if (share < shares) {
+    float z = 0.f;
+    for (int r0 = share; r0 < a.rank; r0 += 4 * shares) {
+      float w[4], m[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int r = min(r0 + i * shares, a.rank - 1);
+        w[i] = a.a2[(size_t)r * a.H * D + hd], m[i] = a.mid[tok * a.ld + r];
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) z = fmaf(r0 + i * shares < a.rank ? w[i] : 0.f, m[i], z);
+    }
+    part[share * D + d] = z;
+  }
+  float bias = 0.f;
+  if (tid < D) {
     qs[d] = a.q[tok * a.ld + hd] * a.q_scale;
     ks[d] = a.k[tok * a.ld + hd];
-    float z = a.a_bias[hd];
-    for (int r = 0; r < a.rank; ++r) z = fmaf(a.a2[(size_t)r * a.H * D + hd], a.mid[tok * a.ld + r], z);
-    gs[d] = expf(-rc_softplus(-z) * a.inv_tau);
+    bias = a.a_bias[hd];
+  }
+  __syncthreads();
+  if (tid < D) {
+    float z = bias;
+    for (int i = 0; i < shares; ++i) z += part[i * D + d];
+    gs[d] = __builtin_amdgcn_exp2f(gla_log2_decay(z, a.inv_tau));
   }
   __syncthreads();
   vec acc = {};
@@ -970,15 +1001,15 @@ gla_step_kernel(GlaArgs a, const float* __restrict__ gain, float eps, const floa
   }
 }
 
-// Prompts in chunks of C = 16 tokens (HDC).  With L_t = the sum of the logarithms of the decays of the chunk's tokens up to
+// Prompts in chunks of C = 16 tokens (HDC).  With L_t = the sum of the (base 2) logarithms of the decays of the chunk's tokens up to
 // t (a vector over the key channels):
-//   o_t = S^T (q_t exp(L_t)) + sum_(j<=t) A_tj v_j,   A_tj = sum_d q_td k_jd exp(L_td - L_jd)
-//   S'  = diag(exp(L_C)) S + sum_j (k_j exp(L_C - L_j)) v_j^T
-// gla_chunks_kernel makes Q exp(L), (K exp(L_C - L))^T, A and exp(L_C) for all chunks side by side; gla_carry_kernel walks a
+//   o_t = S^T (q_t 2^L_t) + sum_(j<=t) A_tj v_j,   A_tj = sum_d q_td k_jd 2^(L_td - L_jd)
+//   S'  = diag(2^L_C) S + sum_j (k_j 2^(L_C - L_j)) v_j^T
+// gla_chunks_kernel makes Q 2^L, (K 2^(L_C - L))^T, A and 2^L_C for all chunks side by side; gla_carry_kernel walks a
 // head's chunks with products alone, in the layout of head_delta_carry_kernel.  None of the exponents above is positive.
-// A on the matrix cores is (Q exp(L)) (K exp(-L))^T, whose second factor grows as the chunk's decays fall: it is taken where
-// no channel loses more than exp(-GLA_SPREAD) within the chunk, and else A is summed term by term.
-#define GLA_SPREAD 60.f
+// A on the matrix cores is (Q 2^L) (K 2^-L)^T, whose second factor grows as the chunk's decays fall: it is taken where
+// no channel loses more than 2^-GLA_SPREAD within the chunk, and else A is summed term by term.
+#define GLA_SPREAD 80.f
 #define GLA_RANK_PIECE 64
 __host__ __device__ __forceinline__ size_t gla_chunk_floats(int NT) { return (size_t)2 * NT * 256 + 256 + 16 * NT; }
 
@@ -995,12 +1026,17 @@ gla_chunks_kernel(GlaArgs a, int n_seqs, float* __restrict__ work, int NT) {
   int first, n;
   if (!hd_chunk_of(blockIdx.x, a.seq_start, n_seqs, first, n)) return;      // (the whole workgroup)
   const int head = blockIdx.y, tid = threadIdx.x, wave = tid / SYN_WAVE, lane = tid % SYN_WAVE, D = a.D;
-  for (int e = tid; e < HDC * DP; e += 256) {
-    const int t = e / DP, d = e % DP;
-    const bool in = t < n && d < D;
-    const size_t at = (size_t)(first + t) * a.ld + head * D + d;
-    qs[t * LDD + d] = in ? a.q[at] * a.q_scale : 0.f;
-    ks[t * LDD + d] = in ? a.k[at] : 0.f;
+  for (int d = lane; d < DP; d += SYN_WAVE) {
+    float q[HDC / 4], k[HDC / 4];
+#pragma unroll
+    for (int i = 0; i < HDC / 4; ++i) {
+      const int t = wave + 4 * i;
+      const bool in = t < n && d < D;
+      const size_t at = (size_t)(first + t) * a.ld + head * D + d;
+      q[i] = in ? a.q[at] * a.q_scale : 0.f, k[i] = in ? a.k[at] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < HDC / 4; ++i) qs[(wave + 4 * i) * LDD + d] = q[i], ks[(wave + 4 * i) * LDD + d] = k[i];
   }
   // the decays: a thread makes one channel's for eight tokens, then the second eight add what the first eight came to
   for (int e0 = 0; e0 < 2 * DP; e0 += 256) {
@@ -1017,16 +1053,24 @@ gla_chunks_kernel(GlaArgs a, int n_seqs, float* __restrict__ work, int NT) {
         mids[(m / nr) * GLA_RANK_PIECE + m % nr] = a.mid[(size_t)(first + min(m / nr, n - 1)) * a.ld + r0 + m % nr];
       __syncthreads();
       if (in)
-        for (int r = 0; r < nr; ++r) {
-          const float w = a.a2[(size_t)(r0 + r) * a.H * D + head * D + d];
+        for (int r = 0; r < nr; r += 8) {
+          float w[8];
 #pragma unroll
-          for (int i = 0; i < 8; ++i) z[i] = fmaf(w, mids[(t0 + i) * GLA_RANK_PIECE + r], z[i]);
+          for (int x = 0; x < 8; ++x)
+            w[x] = r + x < nr ? a.a2[(size_t)(r0 + r + x) * a.H * D + head * D + d] : 0.f;
+#pragma unroll
+          for (int x = 0; x < 8; ++x) {
+            if (r + x < nr) {
+#pragma unroll
+              for (int i = 0; i < 8; ++i) z[i] = fmaf(w[x], mids[(t0 + i) * GLA_RANK_PIECE + r + x], z[i]);
+            }
+          }
         }
     }
     float run = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      run -= (in && t0 + i < n) ? rc_softplus(-z[i]) * a.inv_tau : 0.f;      // (tokens beyond the chunk's: nothing decays)
+      run += (in && t0 + i < n) ? gla_log2_decay(z[i], a.inv_tau) : 0.f;      // (tokens beyond the chunk's: nothing decays)
       z[i] = run;
     }
     if (mine && t0 == 0) {
@@ -1057,19 +1101,19 @@ gla_chunks_kernel(GlaArgs a, int n_seqs, float* __restrict__ work, int NT) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int d = 16 * tile + 4 * g + j, dt = 16 * tile + m, t = 4 * g + j;
-      fq[j] = qs[m * LDD + d] * expf(Ls[m * LDD + d]);
-      ft[j] = ks[t * LDD + dt] * expf(Ls[(HDC - 1) * LDD + dt] - Ls[t * LDD + dt]);
+      fq[j] = qs[m * LDD + d] * __builtin_amdgcn_exp2f(Ls[m * LDD + d]);
+      ft[j] = ks[t * LDD + dt] * __builtin_amdgcn_exp2f(Ls[(HDC - 1) * LDD + dt] - Ls[t * LDD + dt]);
     }
     ((hd_frag*)wf)[e] = fq, ((hd_frag*)wf)[NT * 64 + e] = ft;
     if (on_cores) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int d = 16 * tile + 4 * g + j;
-        acc = hd_mfma(fq[j], ks[m * LDD + d] * expf(-Ls[m * LDD + d]), acc);
+        acc = hd_mfma(fq[j], ks[m * LDD + d] * __builtin_amdgcn_exp2f(-Ls[m * LDD + d]), acc);
       }
     }
   }
-  for (int d = tid; d < DP; d += 256) wf[2 * NT * 256 + 256 + d] = expf(Ls[(HDC - 1) * LDD + d]);
+  for (int d = tid; d < DP; d += 256) wf[2 * NT * 256 + 256 + d] = __builtin_amdgcn_exp2f(Ls[(HDC - 1) * LDD + d]);
   const int t = tid / HDC, j = tid % HDC;
   float A = 0.f;
   if (on_cores) {
@@ -1080,31 +1124,103 @@ gla_chunks_kernel(GlaArgs a, int n_seqs, float* __restrict__ work, int NT) {
     for (int w = 0; w < 4; ++w) A += part[(w * HDC + t) * (HDC + 1) + j];
   } else if (t >= j) {
     for (int d = 0; d < D; ++d)
-      A = fmaf(qs[t * LDD + d] * ks[j * LDD + d], expf(Ls[t * LDD + d] - Ls[j * LDD + d]), A);
+      A = fmaf(qs[t * LDD + d] * ks[j * LDD + d], __builtin_amdgcn_exp2f(Ls[t * LDD + d] - Ls[j * LDD + d]), A);
   }
   wf[2 * NT * 256 + ((j / 4) * 16 + t) * 4 + j % 4] = t >= j ? A : 0.f;      // row t, k = j
 }
 
+// One chunk's operands of a wave that holds rows of the state, and of the wave that makes the outputs.
 template <int TPW, int CG>
-struct GlaOperands {
-  hd_frag q[TPW], kt[TPW], A;
-  f32x4 gc[TPW], v[CG];      // exp(L_C) of the rows 4 g + j, the values of the tokens 4 g + j in this lane's columns
+struct GlaRows {
+  hd_frag q[TPW], kt[TPW];
+  f32x4 gc[TPW], v[CG];      // 2^L_C of the rows 4 g + j, the values of the tokens 4 g + j in this lane's columns
+};
+template <int CG>
+struct GlaOutput {
+  hd_frag A;
+  f32x4 v[CG];
 };
 
 // W waves hold TPW tiles of 16 rows of a head's state each, CG groups of 16 columns a workgroup; one more wave makes and
-// stores the outputs from what the waves' rows give to Q S (through LDS, two buffers in turns: one barrier a chunk).
-template <int TPW, int W, int CG>
+// stores the outputs from what the waves' rows give to Q S (through LDS, two buffers in turns: one barrier a chunk).  The
+// operands are asked for STAGES chunks ahead.
+template <int TPW, int W, int CG, int STAGES>
 __global__ void __launch_bounds__((W + 1) * SYN_WAVE)
 gla_carry_kernel(GlaArgs a, const float* __restrict__ work, float* __restrict__ o) {
   constexpr int NT = TPW * W;
+  static_assert(STAGES == 2 || STAGES == 4, "the two buffers of partial sums follow the chunk's parity");
   __shared__ __attribute__((aligned(16))) f32x4 part[2][W][CG][SYN_WAVE];
   const int head = blockIdx.x, b = blockIdx.z, wave = threadIdx.x / SYN_WAVE, lane = threadIdx.x % SYN_WAVE;
-  const bool holds = wave < W;                       // (else the wave of the outputs)
   const int H = a.H, D = a.D, E = a.E, g = lane / 16, col = blockIdx.y * 16 * CG + lane % 16;
   const int s0 = a.seq_start[b], n_new = a.seq_start[b + 1] - s0;
   if (n_new <= 0) return;                            // (the whole workgroup)
   int slot = a.seq_slot[b];
   if (slot < 0 || slot >= a.state_rows) slot = a.state_rows - 1;
+  const int chunk0 = s0 / HDC + b, n_chunks = (n_new + HDC - 1) / HDC;
+  const float* vp = a.v + (size_t)s0 * a.ld + head * E;
+  auto chunk_of = [&](int c) { return work + ((size_t)(chunk0 + c) * H + head) * gla_chunk_floats(NT); };
+  auto values = [&](f32x4 (&v)[CG], int c) {
+#pragma unroll
+    for (int y = 0; y < CG; ++y)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)      // (tokens beyond the last meet zeros; columns beyond are not stored)
+        v[y][j] = vp[(size_t)min(c * HDC + 4 * g + j, n_new - 1) * a.ld + min(col + 16 * y, E - 1)];
+  };
+  // every wave walks all chunks, with one barrier a chunk
+  auto walk = [&](auto& x0, auto& x1, auto& x2, auto& x3, auto&& ask, auto&& step) {
+    ask(x0, 0), ask(x1, 1);
+    if constexpr (STAGES == 4) ask(x2, 2), ask(x3, 3);
+    for (int c = 0; c < n_chunks; c += STAGES) {
+      step(x0, c, 0);
+      ask(x0, c + STAGES);
+      if (c + 1 < n_chunks) {
+        step(x1, c + 1, 1);
+        ask(x1, c + 1 + STAGES);
+      }
+      if constexpr (STAGES == 4) {
+        if (c + 2 < n_chunks) {
+          step(x2, c + 2, 0);
+          ask(x2, c + 2 + STAGES);
+        }
+        if (c + 3 < n_chunks) {
+          step(x3, c + 3, 1);
+          ask(x3, c + 3 + STAGES);
+        }
+      }
+    }
+  };
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  if (wave == W) {
+    float* op = o + (size_t)s0 * H * E + head * E + col;
+    GlaOutput<CG> x0, x1, x2, x3;
+    walk(x0, x1, x2, x3,
+         [&](GlaOutput<CG>& x, int c) {
+           c = min(c, n_chunks - 1);
+           x.A = ((const hd_frag*)(chunk_of(c) + 2 * NT * 256))[lane];
+           values(x.v, c);
+         },
+         [&](const GlaOutput<CG>& x, int c, int at) {
+           f32x4 out[CG];
+#pragma unroll
+           for (int y = 0; y < CG; ++y) {
+             out[y] = zero;
+#pragma unroll
+             for (int j = 0; j < 4; ++j) out[y] = hd_mfma(x.A[j], x.v[y][j], out[y]);
+           }
+           __syncthreads();
+#pragma unroll
+           for (int y = 0; y < CG; ++y) {
+#pragma unroll
+             for (int w = 0; w < W; ++w) out[y] += part[at][w][y][lane];
+#pragma unroll
+             for (int j = 0; j < 4; ++j) {
+               const int t = c * HDC + 4 * g + j;
+               if (t < n_new && col + 16 * y < E) op[(size_t)t * H * E + 16 * y] = out[y][j];
+             }
+           }
+         });
+    return;
+  }
   float* Sg = a.state + ((size_t)slot * H + head) * D * E;
   f32x4 S[CG][TPW];
 #pragma unroll
@@ -1114,80 +1230,42 @@ gla_carry_kernel(GlaArgs a, const float* __restrict__ work, float* __restrict__ 
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int d = 16 * (wave * TPW + i) + 4 * g + j, c = col + 16 * y;
-        S[y][i][j] = (holds && c < E && d < D) ? Sg[(size_t)d * E + c] : 0.f;
+        S[y][i][j] = (c < E && d < D) ? Sg[(size_t)d * E + c] : 0.f;
       }
-  const int chunk0 = s0 / HDC + b, n_chunks = (n_new + HDC - 1) / HDC;
-  const float* vp = a.v + (size_t)s0 * a.ld + head * E;
-  float* op = o + (size_t)s0 * H * E + head * E + col;
-  auto ask = [&](GlaOperands<TPW, CG>& x, int c) {
-    c = min(c, n_chunks - 1);
-    const float* wf = work + ((size_t)(chunk0 + c) * H + head) * gla_chunk_floats(NT);
-    if (holds) {
-      const hd_frag* kf = (const hd_frag*)wf + wave * TPW * 64 + lane;
+  GlaRows<TPW, CG> x0, x1, x2, x3;
+  walk(x0, x1, x2, x3,
+       [&](GlaRows<TPW, CG>& x, int c) {
+         c = min(c, n_chunks - 1);
+         const float* wf = chunk_of(c);
+         const hd_frag* kf = (const hd_frag*)wf + wave * TPW * 64 + lane;
 #pragma unroll
-      for (int i = 0; i < TPW; ++i) {
-        x.q[i] = kf[i * 64], x.kt[i] = kf[(NT + i) * 64];
-        x.gc[i] = ((const f32x4*)(wf + 2 * NT * 256 + 256))[(wave * TPW + i) * 4 + g];
-      }
-    } else {
-      x.A = ((const hd_frag*)(wf + 2 * NT * 256))[lane];
-    }
+         for (int i = 0; i < TPW; ++i) {
+           x.q[i] = kf[i * 64], x.kt[i] = kf[(NT + i) * 64];
+           x.gc[i] = ((const f32x4*)(wf + 2 * NT * 256 + 256))[(wave * TPW + i) * 4 + g];
+         }
+         values(x.v, c);
+       },
+       [&](const GlaRows<TPW, CG>& x, int c, int at) {
 #pragma unroll
-    for (int y = 0; y < CG; ++y)
+         for (int y = 0; y < CG; ++y) {
+           f32x4 qs[2] = {zero, zero};
 #pragma unroll
-      for (int j = 0; j < 4; ++j)      // (tokens beyond the last meet zeros; columns beyond are not stored)
-        x.v[y][j] = vp[(size_t)min(c * HDC + 4 * g + j, n_new - 1) * a.ld + min(col + 16 * y, E - 1)];
-  };
-  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-  auto step = [&](const GlaOperands<TPW, CG>& x, int c, int at) {
-    if (holds) {
+           for (int i = 0; i < TPW; ++i)
 #pragma unroll
-      for (int y = 0; y < CG; ++y) {
-        f32x4 qs[2] = {zero, zero};
+             for (int j = 0; j < 4; ++j) qs[j & 1] = hd_mfma(x.q[i][j], S[y][i][j], qs[j & 1]);
+           part[at][wave][y][lane] = qs[0] + qs[1];
+         }
+         __syncthreads();
 #pragma unroll
-        for (int i = 0; i < TPW; ++i)
+         for (int y = 0; y < CG; ++y) {
 #pragma unroll
-          for (int j = 0; j < 4; ++j) qs[j & 1] = hd_mfma(x.q[i][j], S[y][i][j], qs[j & 1]);
-        part[at][wave][y][lane] = qs[0] + qs[1];
-      }
-    }
-    __syncthreads();
-    if (holds) {
+           for (int i = 0; i < TPW; ++i) S[y][i] *= x.gc[i];
 #pragma unroll
-      for (int y = 0; y < CG; ++y) {
+           for (int j = 0; j < 4; ++j)
 #pragma unroll
-        for (int i = 0; i < TPW; ++i) S[y][i] *= x.gc[i];
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-#pragma unroll
-          for (int i = 0; i < TPW; ++i) S[y][i] = hd_mfma(x.kt[i][j], x.v[y][j], S[y][i]);
-      }
-    } else {
-#pragma unroll
-      for (int y = 0; y < CG; ++y) {
-        f32x4 out = part[at][0][y][lane];
-#pragma unroll
-        for (int w = 1; w < W; ++w) out += part[at][w][y][lane];
-#pragma unroll
-        for (int j = 0; j < 4; ++j) out = hd_mfma(x.A[j], x.v[y][j], out);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int t = c * HDC + 4 * g + j;
-          if (t < n_new && col + 16 * y < E) op[(size_t)t * H * E + 16 * y] = out[j];
-        }
-      }
-    }
-  };
-  GlaOperands<TPW, CG> even, odd;
-  ask(even, 0), ask(odd, 1);
-  for (int c = 0; c < n_chunks; c += 2) {
-    step(even, c, 0);
-    ask(even, c + 2);
-    if (c + 1 < n_chunks) {
-      step(odd, c + 1, 1);
-      ask(odd, c + 3);
-    }
-  }
+             for (int i = 0; i < TPW; ++i) S[y][i] = hd_mfma(x.kt[i][j], x.v[y][j], S[y][i]);
+         }
+       });
 #pragma unroll
   for (int y = 0; y < CG; ++y)
 #pragma unroll
@@ -1195,7 +1273,7 @@ gla_carry_kernel(GlaArgs a, const float* __restrict__ work, float* __restrict__ 
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int d = 16 * (wave * TPW + i) + 4 * g + j, c = col + 16 * y;
-        if (holds && c < E && d < D) Sg[(size_t)d * E + c] = S[y][i][j];
+        if (c < E && d < D) Sg[(size_t)d * E + c] = S[y][i][j];
       }
 }
 
@@ -1226,7 +1304,7 @@ SYN_EXPORT int syn_gated_linear_scan(const float* q, const float* k, const float
   const int groups = (E + 15) / 16;
   const bool wide = (long)H * n_seqs * ((groups + 1) / 2) >= 2L * syn_compute_units();
   const dim3 grid(H, wide ? (groups + 1) / 2 : groups, n_seqs);
-#define SYN_GLA2(T, W, CG) gla_carry_kernel<T, W, CG><<<grid, (W + 1) * SYN_WAVE, 0, stream>>>(a, scratch, o)
+#define SYN_GLA2(T, W, CG) gla_carry_kernel<T, W, CG, (T) <= 2 ? 4 : 2><<<grid, (W + 1) * SYN_WAVE, 0, stream>>>(a, scratch, o)
 #define SYN_GLA(T, W)                 \
   case T * W:                         \
     if (wide) SYN_GLA2(T, W, 2);      \
@@ -1255,7 +1333,7 @@ SYN_EXPORT int syn_gated_linear_step(const float* q, const float* k, const float
   SYN_CHECK(gain && gate && out && out_ld >= H * E, "gated_linear_step: result rows of %d values", out_ld);
   const bool four = E % 4 == 0 && (uintptr_t)state % 16 == 0;
   const int row_groups = GLA_STEP_THREADS / (four ? E / 4 : E);
-  const size_t bytes = (3 * (size_t)D + (size_t)row_groups * E) * sizeof(float);
+  const size_t bytes = (3 * (size_t)D + (size_t)max(row_groups * E, GLA_STEP_THREADS)) * sizeof(float);
   const dim3 grid(H, n_seqs);
 #define SYN_GLAS(VEC, T) gla_step_kernel<VEC, T><<<grid, GLA_STEP_THREADS, bytes, stream>>>(a, gain, eps, gate, (T*)out, out_ld)
   if (out_is_f32) {

@@ -168,8 +168,8 @@ def _activation_args(activation):
 def embed(table, ids, resid, scale=1.0, sinusoid=None, keep=None):
     """resid[n, :] = scale * table[ids[n], :] as float.  table [V, H] bf16|f32 (or bf16 in fragment order, pack_weight: four
     dimensions), ids [N] int32, resid [N, H] f32.
-    sinusoid = (rates float64 [(H + 1) / 2], positions int32 [N]): sin(p f_i) is added at column 2 i and cos(p f_i) at
-    2 i + 1 for the row's position p.  keep [N, H] f32: receives the same rows as resid."""
+    sinusoid = (rates float64 [(H + 1) / 2] in turns a position, f_i / (2 pi), positions int32 [N]): sin(p f_i) is added at
+    column 2 i and cos(p f_i) at 2 i + 1 for the row's position p.  keep [N, H] f32: receives the same rows as resid."""
     if isinstance(table, torch.Tensor) and table.dim() == 4:
         _need(table, "embed.table", _BF16, (None, None, 64, 8))
         H, kind = table.shape[1] * 32, 2

@@ -13,6 +13,7 @@ same arithmetic on fewer rows.
 """
 from __future__ import annotations
 
+import math
 from dataclasses import dataclass
 
 import torch
@@ -48,7 +49,8 @@ class TokenEmbedding(Part):
         self.table = Matrix(get(self.name))       # (a tied output head multiplies with the same matrix)
         if self.sinusoid_base is not None:
             i = torch.arange((self.hidden + 1) // 2, dtype=torch.float64)
-            self.rates = (float(self.sinusoid_base) ** (-2.0 * i / self.hidden)).to(self.table.device)
+            # (in turns a position)
+            self.rates = (float(self.sinusoid_base) ** (-2.0 * i / self.hidden) / (2.0 * math.pi)).to(self.table.device)
 
     def forward(self, ids, positions=None, keep=None):
         """positions [N] int32: of the rows' tokens (read with sinusoid_base); keep [N, hidden] float: gets the rows too."""
