@@ -43,7 +43,7 @@ class RmsNorm(Part):
     def add_apply(self, resid, delta, out_dtype, rows=None):
         """resid [N, dim] float: with rows None, resid += delta (if any) in place and every row is
         normed; with rows [n] int32 only those rows of resid + delta are normed and resid is kept."""
-        more = (None, None)
+        more = ()
         if isinstance(delta, InjectedDelta):
             # the residual gets rows or a vector beside the last sublayer's result: added in the pass that norms it
             if self.gain_offset == 0.0 and not self._runs_product(resid, delta.inner, out_dtype, rows):
