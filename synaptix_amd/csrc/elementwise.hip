@@ -54,6 +54,7 @@ __global__ void embed_packed_kernel(const bf16* __restrict__ table, const int* _
   float* out = resid + (size_t)n * H;
   for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < H / 8; c += blockDim.x * gridDim.y) {   // values 8 c .. 8 c + 7 of the row
     const bf16x8 v = *(const bf16x8*)(group + (size_t)(c / 4) * 512 + ((c % 4) * 16 + id % 16) * 8);
+    f32x4 x[2];
 #pragma unroll
     for (int e = 0; e < 8; e += 2) {
       float x0 = (float)v[e] * scale, x1 = (float)v[e + 1] * scale;
@@ -62,8 +63,12 @@ __global__ void embed_packed_kernel(const bf16* __restrict__ table, const int* _
         embed_position(p, n, c * 4 + e / 2, s, t);
         x0 += s, x1 += t;
       }
-      out[c * 8 + e] = x0, out[c * 8 + e + 1] = x1;
-      if (keep) keep[(size_t)n * H + c * 8 + e] = x0, keep[(size_t)n * H + c * 8 + e + 1] = x1;
+      x[e / 4][e % 4] = x0, x[e / 4][e % 4 + 1] = x1;
+    }
+    ((f32x4*)out)[2 * c] = x[0], ((f32x4*)out)[2 * c + 1] = x[1];
+    if (keep) {
+      f32x4* k = (f32x4*)(keep + (size_t)n * H);
+      k[2 * c] = x[0], k[2 * c + 1] = x[1];
     }
   }
 }
@@ -79,6 +84,7 @@ SYN_EXPORT int syn_embed(const void* table, int table_kind, const int* ids, floa
     embed_kernel<float><<<n_tokens, 256, 0, stream>>>((const float*)table, ids, resid, H, scale, p, keep);
   } else if (table_kind == 2) {
     SYN_CHECK(H % 32 == 0, "embed: a table in fragment order has a width that is a multiple of 32, not %d", H);
+    SYN_CHECK((uintptr_t)resid % 16 == 0 && (uintptr_t)keep % 16 == 0, "embed: the rows are not aligned");
     const dim3 grid(n_tokens, rates ? (H / 8 + 63) / 64 : 1);
     embed_packed_kernel<<<grid, rates ? 64 : 256, 0, stream>>>((const bf16*)table, ids, resid, H, scale, p, keep);
   } else {
